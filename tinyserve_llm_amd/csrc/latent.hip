@@ -14,6 +14,7 @@
 //   * `ts_paged_attention_latent`: multi-query attention over the cached rows: causal, windowed or chunked
 //     (`ts_first_key`), softmax in 32-bit; keys are visited in chunks of 64 counted from position 0, so the order of
 //     every sum depends on the token's position alone. One workgroup per token; its waves take the heads in turn.
+//     Optionally a learned sink per head in the softmax's denominator and a gate per head (sigmoid) on the result.
 #include "common.h"
 
 #define LT_WAVES 4
@@ -267,7 +268,8 @@ __global__ void __launch_bounds__(LT_THREADS)
 paged_attention_latent_kernel(TO* __restrict__ out, const TQ* __restrict__ q, const TC* __restrict__ cache,
                               const int32_t* __restrict__ block_tables, const int32_t* __restrict__ seq_of_token,
                               const int32_t* __restrict__ positions, int nh, int rank, int row, int page_size, int64_t kp,
-                              int64_t ks, int max_blocks, float scale, int window, int page_run) {
+                              int64_t ks, int max_blocks, float scale, int window, int page_run, const float* __restrict__ sinks,
+                              const float* __restrict__ gate, int64_t gate_token) {
   __shared__ float q_s[LT_WAVES][LT_MAX_ROW];
   __shared__ float p_s[LT_WAVES][TS_WAVE];
   __shared__ int64_t row_s[LT_WAVES][TS_WAVE];             // element offset of each key's cached row
@@ -281,7 +283,8 @@ paged_attention_latent_kernel(TO* __restrict__ out, const TQ* __restrict__ q, co
     wave_sync();
     for (int d = lane; d < row; d += TS_WAVE) q_s[wave][d] = Num<TQ>::ld(qrow + d);
     wave_sync();
-    float m = -INFINITY, l = 0.f;
+    // (a sink is a key of its own score without a value: the sums start with it)
+    float m = sinks ? sinks[h] : -INFINITY, l = sinks ? 1.0f : 0.f;
     float acc[LT_MAX_RANK / TS_WAVE];
 #pragma unroll
     for (int i = 0; i < LT_MAX_RANK / TS_WAVE; ++i) acc[i] = 0.f;
@@ -321,7 +324,7 @@ paged_attention_latent_kernel(TO* __restrict__ out, const TQ* __restrict__ q, co
       wave_sync();
     }
     TO* orow = out + ((int64_t)t * nh + h) * rank;
-    const float inv = 1.0f / l;
+    const float inv = 1.0f / l / (gate ? 1.0f + expf(-gate[(int64_t)t * gate_token + h]) : 1.0f);
 #pragma unroll
     for (int i = 0; i < LT_MAX_RANK / TS_WAVE; ++i) {
       const int d = lane + i * TS_WAVE;
@@ -333,14 +336,16 @@ paged_attention_latent_kernel(TO* __restrict__ out, const TQ* __restrict__ q, co
 extern "C" int ts_paged_attention_latent(void* out, int out_dtype, const void* q, int q_dtype, const void* cache, int cache_dtype,
                                          const int32_t* block_tables, const int32_t* seq_of_token, const int32_t* positions,
                                          int num_tokens, int nh, int rank, int rot, int page_size, int64_t kp, int64_t ks,
-                                         int max_blocks, float scale, int window, int page_run, hipStream_t stream) {
+                                         int max_blocks, float scale, int window, int page_run, const float* sinks,
+                                         const float* gate, int64_t gate_token, hipStream_t stream) {
   if (num_tokens <= 0) return TS_OK;
   if (nh <= 0 || rank <= 0 || rank > LT_MAX_RANK || rot < 0 || rank + rot > LT_MAX_ROW || page_size <= 0 || max_blocks <= 0 ||
       page_run < 0 || page_run > 16)
     return TS_BAD_SHAPE;
 #define LT_ATTEND(TC, TQ, TO) \
   paged_attention_latent_kernel<TC, TQ, TO><<<num_tokens, LT_THREADS, 0, stream>>>((TO*)out, (const TQ*)q, (const TC*)cache, \
-      block_tables, seq_of_token, positions, nh, rank, rank + rot, page_size, kp, ks, max_blocks, scale, window, page_run)
+      block_tables, seq_of_token, positions, nh, rank, rank + rot, page_size, kp, ks, max_blocks, scale, window, page_run, sinks, \
+      gate, gate_token)
   if (cache_dtype == 0 && q_dtype == 0 && out_dtype == 0) LT_ATTEND(float, float, float);
   else if (cache_dtype == 1 && q_dtype == 0 && out_dtype == 1) LT_ATTEND(bf16_t, float, bf16_t);
   else if (cache_dtype == 1 && q_dtype == 0 && out_dtype == 0) LT_ATTEND(bf16_t, float, float);

@@ -14,7 +14,8 @@
 // while the next step's keys and values are on their way. Where a step has few tiles (decoded tokens) the keys of a
 // tile are cut into stretches, a workgroup each, whose parts (maximum, sum, unnormalised rows) a second kernel adds up.
 // Queries arrive 32-bit and are rounded to bfloat16 once, as the keys were. Scores, maxima, weights and sums are
-// 32-bit. Causal, with a sliding window or chunks (`ts_first_key`).
+// 32-bit. Causal, with a sliding window or chunks (`ts_first_key`). Optionally a learned sink per head in the softmax's
+// denominator and a gate per head (sigmoid) on the result.
 #include "attention_mfma.h"
 
 #define LM_WAVES 4
@@ -22,6 +23,16 @@
 #define LM_RT 2                 // 16-row tiles of a workgroup
 #define LM_ROWS (16 * LM_RT)
 #define LM_MAX_SPLITS 16
+
+// What an unnormalised sum is multiplied by: 1 / (its weights' sum `total`, in units of 2^m, and the head's sink's).
+static __device__ __forceinline__ float lm_scale(float m, float total, const float* __restrict__ sinks, int head) {
+  if (!sinks) return 1.0f / total;
+  const float s = sinks[head] * 1.4426950408889634f, top = fmaxf(m, s);
+  return fast_exp2(m - top) / (total * fast_exp2(m - top) + fast_exp2(s - top));
+}
+static __device__ __forceinline__ float lm_gate(const float* __restrict__ gate, int64_t at) {
+  return gate ? 1.0f / (1.0f + expf(-gate[at])) : 1.0f;
+}
 
 // CPW: 32-wide pieces of a cached row per wave (row <= 128 CPW); VPW: 16-wide blocks of value columns per wave
 // (rank <= 64 VPW). Wave w takes pieces w, w + 4, ... and blocks w, w + 4, ...; those past the actual sizes are loaded
@@ -33,7 +44,8 @@ latent_attention_mfma_kernel(TO* __restrict__ out, float* __restrict__ part_o, f
                              const int32_t* __restrict__ block_tables, const int32_t* __restrict__ seq_of_token,
                              const int32_t* __restrict__ positions, const int32_t* __restrict__ tiles, int num_tiles,
                              int tile_tokens, int heads_block, int nh, int rank, int row, int64_t kp, int64_t ks, int64_t vp,
-                             int64_t vd, int max_blocks, float scale_log2, int window, int page_run, int splits) {
+                             int64_t vd, int max_blocks, float scale_log2, int window, int page_run, int splits,
+                             const float* __restrict__ sinks, const float* __restrict__ gate, int64_t gate_token) {
   constexpr int QS = CPW * 128 + 8;                         // a row of the queries in shared memory, skewed
   __shared__ __attribute__((aligned(16))) bf16_t q_s[LM_ROWS][QS];
   __shared__ __attribute__((aligned(16))) float4_t s_part[2][LM_WAVES][LM_RT][2][TS_WAVE];
@@ -217,7 +229,7 @@ latent_attention_mfma_kernel(TO* __restrict__ out, float* __restrict__ part_o, f
     if (tok >= count || tok >= tile_tokens) continue;
     const int64_t item = (int64_t)(t0 + tok) * nh + head;
     if (splits == 1) {
-      const float inv = 1.0f / total;
+      const float inv = lm_scale(m[rt], total, sinks, head) * lm_gate(gate, (int64_t)(t0 + tok) * gate_token + head);
 #pragma unroll
       for (int i = 0; i < VPW; ++i) {
         const int db = wave + LM_WAVES * i;
@@ -246,8 +258,11 @@ latent_attention_mfma_kernel(TO* __restrict__ out, float* __restrict__ part_o, f
 template <typename TO>
 __global__ void __launch_bounds__(LM_THREADS)
 latent_attention_combine_kernel(TO* __restrict__ out, const float* __restrict__ part_o, const float* __restrict__ part_ml,
-                                int rank, int splits) {
+                                int rank, int splits, int nh, const float* __restrict__ sinks, const float* __restrict__ gate,
+                                int64_t gate_token) {
   const int64_t item = blockIdx.x;
+  const int64_t tok = item / nh;
+  const int head = (int)(item - tok * nh);
   const float* ml = part_ml + item * splits * 2;
   float ms[LM_MAX_SPLITS], ls[LM_MAX_SPLITS], top = -INFINITY;
 #pragma unroll
@@ -262,7 +277,7 @@ latent_attention_combine_kernel(TO* __restrict__ out, const float* __restrict__ 
     weight[z] = z < splits ? fast_exp2(ms[z] - top) : 0.f;   // (a stretch without keys: 2^-inf = 0)
     total += weight[z] * ls[z];
   }
-  const float inv = 1.0f / total;
+  const float inv = lm_scale(top, total, sinks, head) * lm_gate(gate, tok * gate_token + head);
   for (int d = threadIdx.x; d < rank; d += LM_THREADS) {
     float part[LM_MAX_SPLITS];
 #pragma unroll
@@ -288,7 +303,8 @@ extern "C" int ts_paged_attention_latent_mfma(void* out, int out_dtype, const fl
                                               const int32_t* tiles, int num_tiles, int tile_tokens, int num_tokens, int nh, int rank,
                                               int rot, int page_size, int64_t kp, int64_t ks, int64_t vp, int64_t vd,
                                               int64_t v_slot, int max_blocks, float scale, int window, int page_run, int splits,
-                                              float* part_o, float* part_ml, hipStream_t stream) {
+                                              float* part_o, float* part_ml, const float* sinks, const float* gate,
+                                              int64_t gate_token, hipStream_t stream) {
   if (num_tiles <= 0 || num_tokens <= 0) return TS_OK;
   const int row = rank + rot;
   const int heads_block = min(nh, LM_ROWS);
@@ -302,15 +318,17 @@ extern "C" int ts_paged_attention_latent_mfma(void* out, int out_dtype, const fl
 #define LM_LAUNCH(CPW, VPW, TO) \
   latent_attention_mfma_kernel<CPW, VPW, TO><<<grid, LM_THREADS, 0, stream>>>((TO*)out, part_o, part_ml, q, (const bf16_t*)k_cache, \
       (const bf16_t*)v_cache, block_tables, seq_of_token, positions, tiles, num_tiles, tile_tokens, heads_block, nh, rank, row, kp, ks, \
-      vp, vd, max_blocks, scale_log2, window, page_run, splits)
+      vp, vd, max_blocks, scale_log2, window, page_run, splits, sinks, gate, gate_token)
 #define LM_PICK(TO) \
   do { \
     if (row <= 256 && rank <= 128) LM_LAUNCH(2, 2, TO); \
     else if (row <= 384 && rank <= 256) LM_LAUNCH(3, 4, TO); \
+    else if (row <= 512) LM_LAUNCH(4, 8, TO); \
     else LM_LAUNCH(5, 8, TO); \
     if (splits > 1) { \
       const int64_t items = (int64_t)num_tokens * nh; \
-      latent_attention_combine_kernel<TO><<<(unsigned)items, LM_THREADS, 0, stream>>>((TO*)out, part_o, part_ml, rank, splits); \
+      latent_attention_combine_kernel<TO><<<(unsigned)items, LM_THREADS, 0, stream>>>((TO*)out, part_o, part_ml, rank, splits, nh, sinks, \
+                                                                                        gate, gate_token); \
     } \
   } while (0)
   if (out_dtype == 0) LM_PICK(float);

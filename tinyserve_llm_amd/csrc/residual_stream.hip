@@ -49,7 +49,7 @@ extern "C" int ts_embedding_stream(float* out, const void* table, const int32_t*
 }
 
 // Row r of the grid: stream row t = rows ? rows[r] : r.
-//   update (a or b given; rows must be null): x[t] += mult * (a[t] + b[t] + bias), written back
+//   update (a, b or bias given; rows must be null): x[t] += mult * (a[t] + b[t] + bias), written back
 //   norms (h1 / h2 given): h[r] = x[t] / sqrt(mean(x[t]^2) + eps) * w, of the updated row
 __global__ void __launch_bounds__(RS_THREADS)
 stream_update_norm_kernel(float* __restrict__ x, const void* __restrict__ a, int a_code, const void* __restrict__ b,
@@ -61,7 +61,7 @@ stream_update_norm_kernel(float* __restrict__ x, const void* __restrict__ a, int
   const int64_t r = blockIdx.x;
   const int64_t t = rows ? rows[r] : r;
   float* xr = x + t * width;
-  const bool update = a || b;
+  const bool update = a || b || bias;
   float squares = 0.f;
   for (int i = threadIdx.x; i < width; i += RS_THREADS) {
     float v = xr[i];
@@ -100,7 +100,7 @@ stream_update_norm_held_kernel(float* __restrict__ x, const float* __restrict__ 
   const int64_t r = blockIdx.x;
   const int64_t t = rows ? rows[r] : r;
   float* xr = x + t * width;
-  const bool update = a || b, bias_on = bias && update;
+  const bool update = a || b || bias, bias_on = bias;
   // an operand that is not there is read from another of its size (the row itself; a norm's weight) and not used
   const float* ar = (a ? a : x) + t * width;
   const float* br = (b ? b : x) + t * width;
@@ -150,7 +150,7 @@ extern "C" int ts_stream_update_norm(float* x, const void* a, int a_dtype, const
                                      const void* w2, int w_dtype, float eps, const int32_t* rows, int num_rows, int width,
                                      hipStream_t stream) {
   if (num_rows <= 0) return TS_OK;
-  if (width <= 0 || !x || (rows && (a || b)) || (h1 && !w1) || (h2 && !w2)) return TS_BAD_SHAPE;
+  if (width <= 0 || !x || (rows && (a || b || bias)) || (h1 && !w1) || (h2 && !w2)) return TS_BAD_SHAPE;
   for (int code : {a_dtype, b_dtype, bias_dtype, h_dtype, w_dtype})
     if (code != 0 && code != 1) return TS_BAD_DTYPE;
   const bool typed = (!a || a_dtype == 0) && (!b || b_dtype == 0) && width <= RS_THREADS * RS_HELD &&
@@ -175,6 +175,64 @@ extern "C" int ts_stream_update_norm(float* x, const void* a, int a_dtype, const
   }
   stream_update_norm_kernel<<<num_rows, RS_THREADS, 0, stream>>>(x, a, a_dtype, b, b_dtype, bias, bias_dtype, mult, h1, h2,
                                                                  h_dtype, w1, w2, w_dtype, eps, rows, width);
+  return ts_check_launch();
+}
+
+// out[t] = [x[t] + a[t] + b[t] | y[t]] (a, b: what branches have left pending, may be absent), rounded to out's storage
+// type: the stream after its sum beside other rows of its width, as a projection's operand. Nothing is written back.
+template <typename TO, bool BY4>
+__global__ void __launch_bounds__(RS_THREADS)
+stream_join_kernel(TO* __restrict__ out, const float* __restrict__ x, const void* __restrict__ a, int a_code,
+                   const void* __restrict__ b, int b_code, const float* __restrict__ y, int64_t items, int width) {
+  for (int64_t idx = (int64_t)blockIdx.x * RS_THREADS + threadIdx.x; idx < items; idx += (int64_t)gridDim.x * RS_THREADS) {
+    constexpr int N = BY4 ? 4 : 1;
+    const int64_t at = idx * N, t = at / width;
+    const int i = (int)(at - t * width);
+    float v[N], w[N];
+    if constexpr (BY4) {                                     // (32-bit branches)
+      const float4 s = *(const float4*)(x + at), o = *(const float4*)(y + at);
+      float4 add = make_float4(0.f, 0.f, 0.f, 0.f);
+      if (a) add = *(const float4*)((const float*)a + at);
+      if (b) {
+        const float4 c = *(const float4*)((const float*)b + at);
+        add.x += c.x; add.y += c.y; add.z += c.z; add.w += c.w;
+      }
+      v[0] = s.x + add.x; v[1] = s.y + add.y; v[2] = s.z + add.z; v[3] = s.w + add.w;
+      w[0] = o.x; w[1] = o.y; w[2] = o.z; w[3] = o.w;
+    } else {
+      float add = 0.f;
+      if (a) add += rs_load(a, a_code, at);
+      if (b) add += rs_load(b, b_code, at);
+      v[0] = x[at] + add;
+      w[0] = y[at];
+    }
+    TO* left = out + t * 2 * width + i;
+    if constexpr (BY4 && sizeof(TO) == 2) {
+      *(uint2*)left = make_uint2((uint32_t)f2bf(v[0]) | ((uint32_t)f2bf(v[1]) << 16), (uint32_t)f2bf(v[2]) | ((uint32_t)f2bf(v[3]) << 16));
+      *(uint2*)(left + width) = make_uint2((uint32_t)f2bf(w[0]) | ((uint32_t)f2bf(w[1]) << 16), (uint32_t)f2bf(w[2]) | ((uint32_t)f2bf(w[3]) << 16));
+    } else {
+#pragma unroll
+      for (int k = 0; k < N; ++k) Num<TO>::st(left + k, v[k]), Num<TO>::st(left + width + k, w[k]);
+    }
+  }
+}
+
+extern "C" int ts_stream_join(void* out, int out_dtype, const float* x, const void* a, int a_dtype, const void* b, int b_dtype,
+                              const float* y, int num_rows, int width, hipStream_t stream) {
+  if (num_rows <= 0) return TS_OK;
+  if (width <= 0) return TS_BAD_SHAPE;
+  for (int code : {out_dtype, a_dtype, b_dtype})
+    if (code != 0 && code != 1) return TS_BAD_DTYPE;
+  const bool by4 = width % 4 == 0 && (!a || a_dtype == 0) && (!b || b_dtype == 0) &&
+                   (((uintptr_t)out | (uintptr_t)x | (uintptr_t)a | (uintptr_t)b | (uintptr_t)y) & 15) == 0;
+  const int64_t items = (int64_t)num_rows * width / (by4 ? 4 : 1);
+  int64_t blocks = (items + RS_THREADS - 1) / RS_THREADS;
+  if (blocks > 16384) blocks = 16384;
+#define RS_JOIN(TO, BY4) \
+  stream_join_kernel<TO, BY4><<<(unsigned)blocks, RS_THREADS, 0, stream>>>((TO*)out, x, a, a_dtype, b, b_dtype, y, items, width)
+  if (out_dtype == 0) { if (by4) RS_JOIN(float, true); else RS_JOIN(float, false); }
+  else { if (by4) RS_JOIN(bf16_t, true); else RS_JOIN(bf16_t, false); }
+#undef RS_JOIN
   return ts_check_launch();
 }
 

@@ -62,6 +62,7 @@ def _bound_tensors(model: DecoderModel):
     """Every parameter tensor the model's parts hold (a tied head's is the embedding's: counted once)."""
     seen: set[int] = set()
     parts = [p for layer in model.layers for p in layer.parts().values()] + [model.embedding, model.head, model.final_norm]
+    parts += list(model.pass_inputs.values())
     for part in parts:
         for name in part.param_specs():
             t = getattr(part, name, None)

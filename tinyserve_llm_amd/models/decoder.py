@@ -47,6 +47,9 @@ class DecoderModel:
         self.final_norm = base.make("norm", spec.final_norm)
         self.position_encodings = {name: base.make("position_encoding", ps)
                                    for name, ps in spec.position_encodings.items()}
+        self.pass_inputs = {name: base.make("pass_input", ps) for name, ps in spec.pass_inputs.items()}
+        if self.pass_inputs and spec.residual_dtype != "float32":
+            raise ValueError("pass inputs work on a 32-bit residual stream (residual_dtype 'float32')")
         sizes = dict(vocab_size=spec.vocab_size, hidden_size=spec.hidden_size, init=spec.embedding_init)
         if spec.residual_dtype not in ("compute", "float32"):
             raise ValueError(f"residual_dtype {spec.residual_dtype!r}: 'compute' or 'float32'")
@@ -66,6 +69,9 @@ class DecoderModel:
         for i, run in enumerate(self.spec.order):
             if not 0 <= run.layer < len(self.layers):
                 raise ValueError(f"order[{i}] names layer {run.layer}, the model has {len(self.layers)}")
+            if run.begins is not None and not (run.begins[0] in self.pass_inputs
+                                               and 0 <= run.begins[1] < self.pass_inputs[run.begins[0]].passes):
+                raise ValueError(f"order[{i}] begins pass {run.begins}, which no pass input of the model makes")
             if run.cache is not None:
                 if not 0 <= run.cache < i:
                     raise ValueError(f"order[{i}] uses the cache of entry {run.cache}, which does not run before it")
@@ -98,7 +104,7 @@ class DecoderModel:
     def graph_safe(self) -> bool:
         """True if every part may be recorded into a HIP graph (see Part.graph_safe)."""
         parts = [p for layer in self.layers for p in layer.parts().values()]
-        parts += [self.final_norm, self.embedding, self.head, *self.position_encodings.values()]
+        parts += [self.final_norm, self.embedding, self.head, *self.position_encodings.values(), *self.pass_inputs.values()]
         return all(getattr(p, "graph_safe", False) for p in parts)
 
     # ---- parameters --------------------------------------------------------------------------
@@ -111,6 +117,9 @@ class DecoderModel:
         for name, enc in self.position_encodings.items():
             for pname, ps in enc.param_specs().items():
                 out[f"positions.{name}.{pname}"] = ps
+        for name, part in self.pass_inputs.items():
+            for pname, ps in part.param_specs().items():
+                out[f"pass_inputs.{name}.{pname}"] = ps
         for pname, ps in self.final_norm.param_specs().items():
             out[f"final_norm.{pname}"] = ps
         for pname, ps in self.head.param_specs().items():
@@ -136,18 +145,22 @@ class DecoderModel:
         for name, enc in self.position_encodings.items():
             enc.bind(grouped.get(f"positions.{name}", {}))
             enc.prepare(device)
+        for name, part in self.pass_inputs.items():
+            part.bind(grouped.get(f"pass_inputs.{name}", {}))
         self.final_norm.bind(grouped.get("final_norm", {}))
 
     def widest_activation(self) -> int:
         """Elements per token of the widest tensor any layer makes (the parts say: `Part.widest_activation`)."""
         return max([self.spec.hidden_size] + [part.widest_activation() for layer in self.layers
-                                              for part in layer.parts().values()])
+                                              for part in layer.parts().values()]
+                   + [part.widest_activation() for part in self.pass_inputs.values()])
 
     def keep_streaming_copies(self) -> int:
         """Lets every part of every layer keep its weights once more in a decode kernel's reading
         order, and the head likewise; returns the bytes that takes."""
         return self.head.keep_streaming_copies() + sum(part.keep_streaming_copies() for layer in self.layers
-                                                       for part in layer.parts().values())
+                                                       for part in layer.parts().values()) \
+            + sum(part.keep_streaming_copies() for part in self.pass_inputs.values())
 
     # ---- one step ----------------------------------------------------------------------------
     def forward(self, ctx: StepContext, memory: list[LayerMemory]) -> tuple[torch.Tensor, torch.Tensor | None]:
@@ -159,9 +172,15 @@ class DecoderModel:
             hidden = enc.on_embedding(hidden, ctx)
         residual = None
         order = self.spec.order
+        # (the layers add to the stream in place: passes that begin later read the embedding's rows from a tensor of their own)
+        start = None
+        if self.pass_inputs:
+            start = hidden.x if order[0].begins is not None and not hidden.pending else self.embedding.forward(ctx).settle()[0]
         for i, (run, mem) in enumerate(zip(order, memory)):
             layer = self.layers[run.layer]
             block = base.BLOCKS[layer.block]
+            if run.begins is not None:
+                hidden = self.pass_inputs[run.begins[0]].forward(hidden, start, ctx, run.begins[1])
             if getattr(block, "first_norm", None) is None:
                 hidden, residual = block(layer, hidden, residual, ctx, mem)
                 continue

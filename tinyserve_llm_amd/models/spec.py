@@ -39,6 +39,9 @@ class LayerRun:
     layer: int
     cache: int | None = None
     store: bool = True
+    # (name, n): this run begins pass number n through a stretch of layers that is run several times; the model's pass
+    # input of that name makes the stream anew right before it
+    begins: tuple[str, int] | None = None
 
 
 @dataclass(frozen=True)
@@ -85,6 +88,8 @@ class ModelSpec:
     # "compute": the residual stream has the engine's storage type; "float32": it is kept in 32-bit
     # floats whatever that type (`parts.stream.ResidualStream`; every block must declare `keeps_stream`)
     residual_dtype: str = "compute"
+    # parts of the "pass_input" family by name: what the runs that begin a pass (`LayerRun.begins`) start from
+    pass_inputs: dict[str, PartSpec] = field(default_factory=dict)
     # what turns token ids into the first hidden rows, and the final rows into logits; None: a
     # plain table and a plain projection (tied to the table if `tie_word_embeddings`)
     embedding: PartSpec | None = None

@@ -101,10 +101,17 @@ def _declare(lib: ctypes.CDLL) -> None:
         "ts_latent_finish": [p, p, i, p, i64, i, i, i, i, i, p, p, f, p, f, p, p, i, i64, i64, p, i64, i64, i, p],
         "ts_latent_mfma_takes": [i, i],
         "ts_heads_gemm_mfma": [p, i, i64, i64, p, i, i64, i64, p, i64, i64, i, i, i, i, p, i64, p],
-        "ts_paged_attention_latent_mfma": [p, i, p, p, p, p, p, p, p, i, i, i, i, i, i, i, i64, i64, i64, i64, i64, i, f, i, i, i, p, p, p],
+        "ts_paged_attention_latent_mfma": [p, i, p, p, p, p, p, p, p, i, i, i, i, i, i, i, i64, i64, i64, i64, i64, i, f, i, i, i, p, p,
+                                           p, p, i64, p],
         "ts_rotate_heads": [p, i, i64, i64, p, i, i64, i64, i, i, i, p, f, p, i, i, p, i64, p],
         "ts_heads_gemm": [p, i, i64, i64, p, i, i64, i64, p, i, i64, i64, i64, i, i, i, i, p, i64, p],
-        "ts_paged_attention_latent": [p, i, p, i, p, i, p, p, p, i, i, i, i, i, i64, i64, i, f, i, i, p],
+        "ts_paged_attention_latent": [p, i, p, i, p, i, p, p, p, i, i, i, i, i, i64, i64, i, f, i, i, p, p, i64, p],
+        "ts_stream_join": [p, i, p, p, i, p, i, p, i, i, p],
+        "ts_ssd_prepare": [p, i, p, p, p, i64, p, p, p, i64, p, p, p, p, p, i, i, i, i, i, i, i, i, i, p],
+        "ts_ssd_conv_keep": [p, i64, p, i64, p, p, i, i, i, i, i, i, i, i, p],
+        "ts_ssd_step": [p, p, i, p, p, p, p, i64, p, p, i, i, i, i, i, i, i, p],
+        "ts_ssd_chunks": [p, p, p, p, p, p, i64, p, p, p, p, p, i, i, i, i, i, i, i, p],
+        "ts_gated_group_norm": [p, i, p, p, i64, p, i, i, i, f, p],
         "ts_mlstm_scan": [p, p, i64, p, p, p, p, p, i, i, i, i, i, f, f, p],
         "ts_mlstm_scan_chunks": [p, p, i64, p, p, p, p, p, p, p, p, p, i, i, i, i, i, f, f, p],
         "ts_mlstm_finish": [p, i, p, p, p, i64, i, i, i, f, i, i, p],
@@ -1640,7 +1647,7 @@ def stream_update_norm(x: torch.Tensor, a: torch.Tensor | None = None, b: torch.
                        rows: torch.Tensor | None = None, out_dtype: torch.dtype = torch.float32
                        ) -> "tuple[torch.Tensor | None, torch.Tensor | None]":
     """The float32 stream x [tokens, width] takes x += mult * (a + b + bias) in place (a, b: what
-    parallel branches made, float32 or bfloat16, either may be None; bias [width] rides on them), and
+    parallel branches made, float32 or bfloat16, either may be None; bias [width] goes to every row), and
     for each given weight norm(x) * weight of the updated rows comes back in `out_dtype` (both norms
     share the row's mean square). With `rows` (int32) nothing is updated and only those rows are
     normalised, in that order."""
@@ -1649,9 +1656,8 @@ def stream_update_norm(x: torch.Tensor, a: torch.Tensor | None = None, b: torch.
     tokens, width = x.shape
     for name, t in (("a", a), ("b", b)):
         _need(t is None or (t.shape == x.shape and t.is_contiguous()), lambda: f"{name} must match the stream")
-    _need(bias is None or (bias.shape == (width,) and bias.is_contiguous() and (a is not None or b is not None)),
-          "a bias is [width] and rides on a branch")
-    _need(rows is None or (a is None and b is None), "picked rows are normalised, not updated")
+    _need(bias is None or (bias.shape == (width,) and bias.is_contiguous()), "a bias is [width]")
+    _need(rows is None or (a is None and b is None and bias is None), "picked rows are normalised, not updated")
     n = tokens
     if rows is not None:
         _need(rows.dtype == torch.int32 and rows.dim() == 1 and rows.is_contiguous(), "rows must be int32")
@@ -1665,6 +1671,20 @@ def stream_update_norm(x: torch.Tensor, a: torch.Tensor | None = None, b: torch.
         _ptr(bias), 0 if bias is None else _code(bias.dtype), float(mult), _ptr(outs[0]), _ptr(outs[1]), _code(out_dtype),
         _ptr(weights[0]), _ptr(weights[1]), _code(given[0].dtype) if given else 0, float(eps), _ptr(rows), n, width, _stream()))
     return outs[0], outs[1]
+
+
+def stream_join(x: torch.Tensor, a: torch.Tensor | None, b: torch.Tensor | None, y: torch.Tensor, out_dtype: torch.dtype) -> torch.Tensor:
+    """[x + a + b | y] row by row as `out_dtype` [tokens, 2 width]: the float32 stream x after its pending sum (a, b float32
+    or bfloat16, either may be None) beside float32 rows y of the same width. Nothing is written back."""
+    _gpu(x, a, b, y)
+    for name, t in (("x", x), ("y", y)):
+        _need(t.dtype == torch.float32 and t.dim() == 2 and t.is_contiguous() and t.shape == x.shape, lambda: f"{name} must be contiguous float32 [tokens, width]")
+    for name, t in (("a", a), ("b", b)):
+        _need(t is None or (t.shape == x.shape and t.is_contiguous()), lambda: f"{name} must match the stream")
+    out = torch.empty((x.shape[0], 2 * x.shape[1]), dtype=out_dtype, device=x.device)
+    _run("stream_join", library().ts_stream_join(_ptr(out), _code(out_dtype), _ptr(x), _ptr(a), 0 if a is None else _code(a.dtype), _ptr(b),
+                                                 0 if b is None else _code(b.dtype), _ptr(y), x.shape[0], x.shape[1], _stream()))
+    return out
 
 
 ACTIVATIONS = {"none": 0, "relu2": 1, "gelu_tanh": 2, "silu": 3, "tanh": 4}
@@ -2266,15 +2286,18 @@ def latent_mfma_takes(q: torch.Tensor, cache: torch.Tensor, v_cache: torch.Tenso
 
 
 def paged_attention_latent(q: torch.Tensor, cache: torch.Tensor, rank: int, ctx, space: int, scale: float, window: int = 0,
-                           chunk_mask: int = 0, out_dtype: torch.dtype | None = None, v_cache: torch.Tensor | None = None
-                           ) -> torch.Tensor:
+                           chunk_mask: int = 0, out_dtype: torch.dtype | None = None, v_cache: torch.Tensor | None = None,
+                           sinks: torch.Tensor | None = None, head_gate: torch.Tensor | None = None) -> torch.Tensor:
     """Multi-query attention of a packed step over cached rows [c | r] (c the first `rank` numbers, which are also
     the values): q [tokens, heads, rank + rot] (float32, or the cache's type), out [tokens, heads, rank] = the softmax
     weights' sum of c. Causal, with a sliding `window` or chunks (`chunk_mask`) as `paged_attention` has them. With
     `v_cache` (the values once more, [pages, page_size, 1, rank], transposed inside a page) bfloat16 caches of the
     sizes it serves go to the matrix-core kernel; everything else, float32 always, to a kernel that is 32-bit
-    throughout and whose sums depend on the token's position alone."""
-    _gpu(q, cache, v_cache)
+    throughout and whose sums depend on the token's position alone. `sinks` (float32 [heads]): exp(sinks[h]) joins the
+    softmax's denominator. `head_gate` (float32 [tokens, heads], rows may lie apart): out is multiplied by sigmoid of it."""
+    _gpu(q, cache, v_cache, sinks, head_gate)
+    _check_head_vectors(q.shape[1], sinks)
+    gate_stride = _check_gate(head_gate, q.shape[0], q.shape[1])
     _need(chunk_mask >= 0 and window >= 0 and not (chunk_mask and window), "a sliding window or chunks, both counted in positions")
     T, H, row = q.shape
     _need(q.is_contiguous() and 0 < rank <= min(row, LATENT_MAX_RANK) and row <= LATENT_MAX_ROW,
@@ -2311,12 +2334,12 @@ def paged_attention_latent(q: torch.Tensor, cache: torch.Tensor, rank: int, ctx,
             _ptr(out), _code(out.dtype), _ptr(q), _ptr(cache), _ptr(v_cache), _ptr(tables), _ptr(ctx.seq_of_token), _ptr(ctx.positions),
             _ptr(tiles), num_tiles, tile_tokens if tiles is not None else 1, T, H, rank, row - rank, cache.shape[1], cache.stride(0),
             cache.stride(1), v_cache.stride(0), v_cache.stride(3), v_cache.stride(1), tables.shape[1], float(scale), mask,
-            _page_run(table_page // cache.shape[1]), splits, _ptr(part_o), _ptr(part_ml), _stream()))
+            _page_run(table_page // cache.shape[1]), splits, _ptr(part_o), _ptr(part_ml), _ptr(sinks), _ptr(head_gate), gate_stride, _stream()))
         return out
     _run("paged_attention_latent", library().ts_paged_attention_latent(
         _ptr(out), _code(out.dtype), _ptr(q), _code(q.dtype), _ptr(cache), _code(cache.dtype), _ptr(tables), _ptr(ctx.seq_of_token),
         _ptr(ctx.positions), T, H, rank, row - rank, cache.shape[1], cache.stride(0), cache.stride(1), tables.shape[1], float(scale),
-        mask, _page_run(table_page // cache.shape[1]), _stream()))
+        mask, _page_run(table_page // cache.shape[1]), _ptr(sinks), _ptr(head_gate), gate_stride, _stream()))
     return out
 
 
@@ -2552,3 +2575,154 @@ def qkv_prepare(qkv: torch.Tensor, positions: torch.Tensor, num_heads: int, num_
         _check_freqs(value_freqs, value_dim)
     _run("qkv_prepare", library().ts_qkv_prepare(_ptr(qkv), _ptr(positions), T, num_heads, num_kv_heads, head_dim, value_dim, _ptr(q_weight),
                                                  _ptr(k_weight), float(eps), _ptr(value_freqs), int(value_interleaved), _stream()))
+
+
+# ---- a state-space mixer with one decay per head ----
+
+SSD_MAX_STATE = 512       # rows of a head's state
+SSD_CHUNK = 64            # tokens of a chunk of the chunked form,
+SSD_CHUNKS_FROM = 24      # which takes the requests of a step that feed at least this many tokens (bfloat16 only)
+
+
+class SsdSizes:
+    """Sizes of a state-space mixer and the padded places its kernels work on: a head's channels in `vp` (a multiple of 16),
+    a group's state rows in `np` (a multiple of 32); a token's mixed row is heads vp | groups np | groups np (x, B, C)."""
+
+    def __init__(self, heads: int, vdim: int, groups: int, state: int, taps: int) -> None:
+        _need(min(heads, vdim, groups, state) > 0 and heads % groups == 0, "positive sizes, heads that divide into the groups")
+        _need(state <= SSD_MAX_STATE and 1 <= taps <= CONV_MAX_TAPS, lambda: f"a state of up to {SSD_MAX_STATE} rows, 1 to {CONV_MAX_TAPS} taps")
+        self.heads, self.vdim, self.groups, self.state, self.taps = heads, vdim, groups, state, taps
+        self.vp, self.np = -(-vdim // 16) * 16, -(-state // 32) * 32
+        self.row = heads * self.vp + 2 * groups * self.np
+        self.inner, self.channels = heads * vdim, heads * vdim + 2 * groups * state
+        self.projected = self.inner + self.channels + heads          # z | x | B | C | dt
+        self.matrix = heads * self.vp * self.np                      # floats of a request's S,
+        self.kept = (taps - 1) * self.row                            # and of the convolution's last inputs behind it
+
+    def spread(self, t: torch.Tensor) -> torch.Tensor:
+        """Something per channel ([channels, ...]) in the places of a mixed row ([row, ...]), zeros in the others."""
+        rest = t.shape[1:]
+        x, b, c = t.split([self.inner, self.groups * self.state, self.groups * self.state])
+        out = torch.zeros((self.row, *rest), dtype=t.dtype, device=t.device)
+        at = self.heads * self.vp
+        out[:at].view(self.heads, self.vp, *rest)[:, :self.vdim] = x.reshape(self.heads, self.vdim, *rest)
+        for part in (b, c):
+            out[at:at + self.groups * self.np].view(self.groups, self.np, *rest)[:, :self.state] = part.reshape(self.groups, self.state, *rest)
+            at += self.groups * self.np
+        return out
+
+
+def _check_ssd_state(state: torch.Tensor, sizes: SsdSizes) -> None:
+    _need(state.dtype == torch.float32 and state.dim() == 2 and state.shape[1] >= sizes.matrix + sizes.kept and state.stride(1) == 1
+          and state.stride(0) % 4 == 0 and state.data_ptr() % 16 == 0,
+          lambda: f"the state must be float32 [slots, >= {sizes.matrix + sizes.kept}], rows at 16-byte borders")
+
+
+def _check_step_requests(ctx) -> None:
+    for name, t, n in (("seq_of_token", ctx.seq_of_token, ctx.num_tokens), ("cu_seqlens", ctx.cu_seqlens, ctx.num_seqs + 1),
+                       ("state_slots", ctx.state_slots, ctx.num_seqs)):
+        _need(t.dtype == torch.int32 and t.shape == (n,) and t.is_contiguous(), lambda: f"{name} must be int32 [{n}]")
+
+
+def ssd_prepare(proj: torch.Tensor, conv_w: torch.Tensor, conv_b: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor,
+                state: torch.Tensor, ctx, sizes: SsdSizes, out_dtype: torch.dtype) -> "tuple[torch.Tensor, torch.Tensor, torch.Tensor]":
+    """From projected rows (float32 [tokens, >= projected], z | x | B | C | dt leading) to (mixed rows [tokens, row] of
+    `out_dtype`: x, B and C through the causal convolution with bias and silu; step sizes softplus(dt + dt_bias) and log
+    decays -exp(a_log) times them, float32 [tokens, heads]). conv_w float32 [taps, row] and conv_b float32 [row] in the
+    places of a mixed row (`SsdSizes.spread`). The rows ahead of a request's first token of the step come from its slot of
+    `state` (float32 [slots, >= matrix + kept], the convolution's inputs behind S), where the step leaves its own last ones."""
+    _gpu(proj, conv_w, conv_b, dt_bias, a_log, state)
+    T, z = proj.shape[0], sizes
+    _need(proj.dtype == torch.float32 and proj.dim() == 2 and proj.is_contiguous() and proj.shape[1] >= z.projected,
+          lambda: f"the projected rows must be contiguous float32 [tokens, >= {z.projected}]")
+    _need(conv_w.dtype == torch.float32 and conv_w.shape == (z.taps, z.row) and conv_w.is_contiguous(), lambda: f"conv_w must be float32 [{z.taps}, {z.row}]")
+    _need(conv_b.dtype == torch.float32 and conv_b.shape == (z.row,) and conv_b.is_contiguous(), lambda: f"conv_b must be float32 [{z.row}]")
+    _check_head_vectors(z.heads, dt_bias, a_log)
+    _check_ssd_state(state, z)
+    _check_step_requests(ctx)
+    _need(ctx.num_tokens == T, "the projected rows are the step's")
+    mixed = torch.empty((T, z.row), dtype=out_dtype, device=proj.device)
+    steps = torch.empty((T, z.heads), dtype=torch.float32, device=proj.device)
+    logs = torch.empty_like(steps)
+    kept = state.data_ptr() + 4 * z.matrix
+    # (a request's only token of the step moves its slot on by itself: nobody else reads it)
+    moves = z.taps > 1 and T == ctx.num_seqs and ctx.max_query_len == 1
+    _run("ssd_prepare", library().ts_ssd_prepare(
+        _ptr(mixed), _code(out_dtype), _ptr(steps), _ptr(logs), _ptr(proj), proj.shape[1], _ptr(conv_w), _ptr(conv_b), kept, state.stride(0),
+        _ptr(dt_bias), _ptr(a_log), _ptr(ctx.cu_seqlens), _ptr(ctx.seq_of_token), _ptr(ctx.state_slots), T, z.heads, z.vdim, z.vp, z.groups,
+        z.state, z.np, z.taps, int(moves), _stream()))
+    if z.taps > 1 and not moves:
+        _run("ssd_conv_keep", library().ts_ssd_conv_keep(
+            kept, state.stride(0), _ptr(proj), proj.shape[1], _ptr(ctx.cu_seqlens), _ptr(ctx.state_slots), ctx.num_seqs, z.heads, z.vdim, z.vp,
+            z.groups, z.state, z.np, z.taps, _stream()))
+    return mixed, steps, logs
+
+
+def ssd_chunk_lists(host_cu_seqlens: list[int], from_tokens: int) -> tuple[list[int], list[int]]:
+    """The chunks of the requests of a packed step that feed at least `from_tokens` tokens: ([(first token, tokens, request,
+    1 if the request's last)...] flattened, [first chunk of each request..., number of chunks])."""
+    flat: list[int] = []
+    cu = [0]
+    for s in range(len(host_cu_seqlens) - 1):
+        a, b = host_cu_seqlens[s], host_cu_seqlens[s + 1]
+        if b - a >= from_tokens:
+            for t in range(a, b, SSD_CHUNK):
+                flat += (t, min(SSD_CHUNK, b - t), s, int(t + SSD_CHUNK >= b))
+        cu.append(len(flat) // 4)
+    return flat, cu
+
+
+def ssd_scan(mixed: torch.Tensor, steps: torch.Tensor, logs: torch.Tensor, skip: torch.Tensor, state: torch.Tensor, ctx,
+             sizes: SsdSizes, chunks_from: int = SSD_CHUNKS_FROM) -> torch.Tensor:
+    """The recurrence over a packed step: per head S <- exp(log) S + step x B^T, y = S C + skip x, each request from and to
+    its slot of `state` (S [heads, vp, np] at the start of the slot's row). mixed, steps, logs as `ssd_prepare` leaves
+    them, skip float32 [heads]. Returns y float32 [tokens, heads vdim]. In bfloat16, requests that feed at least
+    `chunks_from` tokens are worked in chunks on the matrix cores; all others, and 32-bit rows always, token by token."""
+    _gpu(mixed, steps, logs, skip, state)
+    z, T = sizes, mixed.shape[0]
+    _need(mixed.shape == (T, z.row) and mixed.is_contiguous(), lambda: f"the mixed rows must be contiguous [tokens, {z.row}]")
+    for t in (steps, logs):
+        _need(t.dtype == torch.float32 and t.shape == (T, z.heads) and t.is_contiguous(), "steps and logs must be float32 [tokens, heads]")
+    _check_head_vectors(z.heads, skip)
+    _check_ssd_state(state, z)
+    _check_step_requests(ctx)
+    _need(ctx.num_tokens == T and chunks_from >= 1, "the mixed rows are the step's")
+    S = ctx.num_seqs
+    out = torch.empty((T, z.inner), dtype=torch.float32, device=mixed.device)
+    chunked = mixed.dtype == torch.bfloat16 and ctx.max_query_len >= chunks_from
+    if chunked:
+        kept = ctx.scratch.get(("ssd_chunks", chunks_from))
+        if kept is None:
+            # (a list copied from the host while a graph is being recorded would be read again, from memory long freed, at every replay)
+            _need(not torch.cuda.is_current_stream_capturing(), "the chunk list is made before a graph is recorded")
+            _need(len(ctx.host_cu_seqlens) == S + 1 and ctx.host_cu_seqlens[-1] == T, "the host's lengths are the step's")
+            flat, cu = ssd_chunk_lists(ctx.host_cu_seqlens, chunks_from)
+            kept = (torch.tensor(flat, dtype=torch.int32).view(-1, 4).to(mixed.device, non_blocking=True),
+                    torch.tensor(cu, dtype=torch.int32).to(mixed.device, non_blocking=True))
+            ctx.scratch[("ssd_chunks", chunks_from)] = kept
+        chunks, chunk_cu = kept
+        C = chunks.shape[0]
+        buf = torch.empty((C, z.matrix), dtype=torch.float32, device=mixed.device)
+        totals = torch.empty((C, z.heads), dtype=torch.float32, device=mixed.device)
+        _run("ssd_chunks", library().ts_ssd_chunks(
+            _ptr(out), _ptr(mixed), _ptr(steps), _ptr(logs), _ptr(skip), _ptr(state), state.stride(0), _ptr(chunks), _ptr(chunk_cu),
+            _ptr(ctx.state_slots), _ptr(buf), _ptr(totals), C, S, z.heads, z.vdim, z.vp, z.groups, z.np, _stream()))
+        if all(b - a >= chunks_from for a, b in zip(ctx.host_cu_seqlens, ctx.host_cu_seqlens[1:])):
+            return out
+    _run("ssd_step", library().ts_ssd_step(
+        _ptr(out), _ptr(mixed), _code(mixed.dtype), _ptr(steps), _ptr(logs), _ptr(skip), _ptr(state), state.stride(0), _ptr(ctx.cu_seqlens),
+        _ptr(ctx.state_slots), S, z.heads, z.vdim, z.vp, z.groups, z.np, chunks_from - 1 if chunked else 0, _stream()))
+    return out
+
+
+def gated_group_norm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, parts: int, eps: float, out_dtype: torch.dtype) -> torch.Tensor:
+    """y silu(gate) (float32 [tokens, width]; the gate's rows may lie apart), cut into `parts` equal parts, each divided by
+    its own root mean square (eps inside the root), times `weight` (float32 [width]), as `out_dtype`."""
+    _gpu(y, gate, weight)
+    T, width = y.shape
+    _need(y.dtype == torch.float32 and y.is_contiguous() and parts > 0 and width % parts == 0, "y must be contiguous float32 [tokens, width], width in equal parts")
+    _need(weight.dtype == torch.float32 and weight.shape == (width,) and weight.is_contiguous(), "the weight must be float32 [width]")
+    out = torch.empty((T, width), dtype=out_dtype, device=y.device)
+    _run("gated_group_norm", library().ts_gated_group_norm(_ptr(out), _code(out_dtype), _ptr(y), _ptr(gate), _check_gate(gate, T, width), _ptr(weight),
+                                                           T, width, parts, float(eps), _stream()))
+    return out

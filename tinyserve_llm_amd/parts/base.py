@@ -212,6 +212,18 @@ class TokenInput(Part):
         raise NotImplementedError
 
 
+class PassInput(Part):
+    """What a pass through a stretch of layers that runs several times starts from: `forward(stream, start, ctx, n)` takes
+    the 32-bit residual stream as the run before left it (`parts.stream.ResidualStream`; used up by the call), the rows the
+    embedding gave (float32, not to be written) and the number of the pass, and returns the stream that the pass's first
+    layer takes. `passes`: how many passes the part has parameters for."""
+
+    passes = 0
+
+    def forward(self, stream, start: torch.Tensor, ctx: StepContext, n: int):
+        raise NotImplementedError
+
+
 class Embedding(Part):
     """Token ids to the first hidden rows [tokens, hidden]."""
 
@@ -247,11 +259,12 @@ POSITION_ENCODINGS: dict[str, Callable[..., PositionEncoding]] = {}
 EMBEDDINGS: dict[str, Callable[..., Embedding]] = {}
 HEADS: dict[str, Callable[..., Head]] = {}
 TOKEN_INPUTS: dict[str, Callable[..., TokenInput]] = {}
+PASS_INPUTS: dict[str, Callable[..., PassInput]] = {}
 BLOCKS: dict[str, Callable[..., Any]] = {}
 
 _TABLES = {"mixer": MIXERS, "feed_forward": FEED_FORWARDS, "norm": NORMS,
            "position_encoding": POSITION_ENCODINGS, "embedding": EMBEDDINGS, "head": HEADS, "block": BLOCKS,
-           "token_input": TOKEN_INPUTS}
+           "token_input": TOKEN_INPUTS, "pass_input": PASS_INPUTS}
 
 
 def register(family: str, name: str) -> Callable:

@@ -135,6 +135,21 @@ def parallel_block(layer: Layer, hidden, residual, ctx: StepContext, mem: LayerM
     return ResidualStream(x, a, b, bias, float(layer.block_args.get("residual_mult", 1.0))), None
 
 
+@register("block", "parallel_one_norm")
+@uses_norms("norm1")
+@keeps_stream
+def parallel_one_norm_block(layer: Layer, hidden, residual, ctx: StepContext, mem: LayerMemory):
+    """x <- x + (mixer(norm1(x)) + feed_forward(norm1(x))): one norm, whose rows both branches read. The stream is 32-bit;
+    both branches' rows are left pending in it, so that the kernel that adds them makes the next layer's norm (or the
+    model's last) as well."""
+    from tinyserve_llm_amd.parts.stream import ResidualStream
+    if not isinstance(hidden, ResidualStream) or residual is not None:
+        raise TypeError("this arrangement runs on a 32-bit residual stream (ModelSpec.residual_dtype = 'float32')")
+    x, h = hidden.take(layer.norms["norm1"])
+    a = layer.mixer.forward(h, ctx, mem)
+    return ResidualStream(x, a, layer.feed_forward.forward(h, ctx)), None
+
+
 @register("block", "sandwich")
 @uses_norms("norm1", "norm1b")
 @keeps_stream

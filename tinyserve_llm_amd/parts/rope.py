@@ -71,16 +71,24 @@ class RotaryFrequencies(PositionEncoding):
 
     graph_safe = True
 
-    def __init__(self, rotary_dim: int, theta: float, interleaved: bool = True, ramp: dict | None = None) -> None:
+    def __init__(self, rotary_dim: int, theta: float, interleaved: bool = True, ramp: dict | None = None, bands: dict | None = None) -> None:
         """`ramp` (factor s, original length L, fast, slow): frequencies are slowed down by s along a ramp over
         the pairs: with d(t) = rotary_dim ln(L / (2 pi t)) / (2 ln theta), lo = max(floor d(fast), 0),
         hi = min(ceil d(slow), rotary_dim - 1) and r_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), pair i
         turns with f_i / s * r_i + f_i (1 - r_i), and cosine and sine are multiplied by `amplitude` =
-        0.1 ln s + 1 (the mixers' kernels take it beside the frequencies)."""
+        0.1 ln s + 1 (the mixers' kernels take it beside the frequencies). `bands` (instead; factor s, low, high,
+        original length L): by wavelength l = 2 pi / f, frequencies with l < L / high stay, those with l > L / low become
+        f / s, those between (1 - m) f / s + m f with m = (L / l - low) / (high - low); no amplitude."""
+        if ramp and bands:
+            raise ValueError("frequencies slow down along a ramp or in bands, not both")
         if rotary_dim % 2 or rotary_dim < 0:
             raise ValueError(f"rotary_dim {rotary_dim}: an even number of dimensions turns")
         self.rotary_dim, self.theta, self.interleaved = rotary_dim, float(theta), interleaved
         self.ramp = dict(ramp) if ramp else None
+        self.bands = dict(bands) if bands else None
+        if self.bands is not None and not (min(self.bands[k] for k in ("factor", "low", "original")) > 0
+                                           and self.bands["high"] >= self.bands["low"]):
+            raise ValueError("frequency bands need positive factor, low and original, and high of at least low")
         if self.ramp is not None and not (self.ramp["factor"] > 0 and self.ramp["original"] > 0 and self.ramp["fast"] > 0
                                           and self.ramp["slow"] > 0 and self.theta > 1):
             raise ValueError("a frequency ramp needs positive factor, original, fast and slow, and a base above 1")
@@ -90,6 +98,12 @@ class RotaryFrequencies(PositionEncoding):
     def host_frequencies(self) -> torch.Tensor:
         i = torch.arange(self.rotary_dim // 2, dtype=torch.float64)
         f = torch.pow(torch.tensor(self.theta, dtype=torch.float64), -2.0 * i / max(1, self.rotary_dim))
+        if self.bands is not None:
+            b = self.bands
+            turns = b["original"] * f / (2.0 * math.pi)              # L / l: the turns a pair makes over L positions
+            mix = (turns - b["low"]) / max(b["high"] - b["low"], 1e-300)
+            between = (1.0 - mix) * f / b["factor"] + mix * f
+            return torch.where(turns > b["high"], f, torch.where(turns < b["low"], f / b["factor"], between))
         if self.ramp is None:
             return f
         r = self.ramp

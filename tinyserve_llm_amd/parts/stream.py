@@ -15,8 +15,9 @@ from tinyserve_llm_amd.ops import hip
 
 class ResidualStream:
     """x [tokens, hidden] float32 and, pending, x += mult * (a + b + bias): `a`, `b` the outputs of a
-    layer's branches (float32 or the engine's storage type; either may be None), `bias` [hidden] a
-    bias that the last projection of a branch left to the sum. With `post` (a norm; then only `a` is
+    layer's branches (float32 or the engine's storage type; either may be None), `bias` [hidden] a row
+    that goes to every token: a bias that the last projection of a branch left to the sum, or a vector that
+    is added to the stream itself. With `post` (a norm; then only `a` is
     pending and `mult` is 1) the pending update is x += post(a), or x += post(a) * scale with `scale`
     (float32 [hidden], a learned factor per channel; with an RMS norm as `post` only)."""
 
@@ -43,6 +44,14 @@ class ResidualStream:
             return out
         self.a, self.post = self.post(self.a)[0], None
         return None
+
+    def joined_with(self, other: torch.Tensor, dtype: torch.dtype) -> torch.Tensor:
+        """[x | other] in `dtype`, x after the pending sum and `other` float32 rows of the same width: a projection's operand.
+        The sum is not kept: this uses the stream up."""
+        self._apply_post()
+        if self.bias is not None or self.mult != 1.0:
+            self.settle()
+        return hip.stream_join(self.x, self.a, self.b, other, dtype)
 
     def rows_as(self, dtype: torch.dtype) -> "tuple[torch.Tensor, torch.Tensor]":
         """Does the pending sum and returns (x, x in `dtype`): the stream's rows as a projection's operand."""
@@ -81,7 +90,7 @@ class ResidualStream:
 
     @property
     def pending(self) -> bool:
-        return self.a is not None or self.b is not None
+        return self.a is not None or self.b is not None or self.bias is not None
 
     def settle(self, weights: "tuple[torch.Tensor | None, torch.Tensor | None]" = (None, None), eps: float = 0.0,
                out_dtype: torch.dtype = torch.float32) -> "tuple[torch.Tensor, torch.Tensor | None, torch.Tensor | None]":
