@@ -187,3 +187,41 @@ def tegolix_configs():
         L("parallel", t_wide, None), L("gla", G(heads=4, dim=32, vdim=32, tau=9.0, decay_rank=12), E(experts=2, identity=5, top=1, ff=48, shared_ff=64)),
         L("parallel", t_short, D(320)), L("gla", G(heads=2, dim=128, vdim=64, tau=20.0, decay_rank=6), D(192))))
     return {"P": (P, 3), "Q": (Q, 4), "R": (R_, 5), "S": (S, 6), "T": (T, 7)}
+
+
+def morulix_configs():
+    """Small Morulix configurations that differ from each other in every size and option: the order of the three mixers,
+    key/value grouping, key and value head sizes (equal or not), how much of a head turns (all, part, none), frequency
+    bands or none, windows (one position, shorter and longer than a page, none), latents larger and smaller than the
+    heads they feed, state-space heads of one group or a group each, of channels and state rows that are multiples of
+    nothing or of several workgroups' slices, taps from one to six, parts of the gated norm that are heads, several heads
+    or pieces of one, a looped stretch at the start, in the middle, over everything, of one layer, run once up to three
+    times, or none, layers with and without a feed-forward, and widths that are multiples of nothing."""
+    from tinyserve_llm_amd.config.morulix import FrequencyBands as Bands, MorulixAttention as A, MorulixConfig, \
+        MorulixLatentAttention as LA, MorulixLayer as L, MorulixMamba2 as M, MorulixRotation as Rot
+    p_att = A(heads=4, kv_heads=2, dim=32, vdim=48, scale=0.3, rot=Rot(16, 10000.0, Bands(3.0, 1.0, 4.0, 64.0)), window=24)
+    P = MorulixConfig(vocab=200, width=80, norm_eps=1e-6, loop_start=1, loop_stop=3, loop_times=3, layers=(
+        L("mamba2", M(heads=4, vdim=20, state=24, groups=2, conv=4, norm_groups=5), 96), L("attention", p_att, 72),
+        L("latent_attention", LA(heads=3, dim=24, vdim=20, kv_rank=40, scale=0.2), 64), L("attention", p_att, None)))
+    Q = MorulixConfig(vocab=131, width=48, norm_eps=1e-4, loop_start=0, loop_stop=2, loop_times=1, layers=(
+        L("attention", A(heads=2, kv_heads=2, dim=16, vdim=16, scale=0.25, rot=Rot(16, 700.0), window=1), 64),
+        L("mamba2", M(heads=1, vdim=16, state=16, groups=1, conv=2, norm_groups=1), None),
+        L("latent_attention", LA(heads=2, dim=16, vdim=16, kv_rank=16, scale=0.4), 40),
+        L("attention", A(heads=4, kv_heads=1, dim=8, vdim=24, scale=0.35, rot=Rot(0, 1.0), window=0), 20),
+        L("mamba2", M(heads=6, vdim=8, state=32, groups=6, conv=1, norm_groups=6), 36)))
+    # sizes that are multiples of nothing in particular: no kernel's fast path takes them
+    R = MorulixConfig(vocab=77, width=99, norm_eps=1e-5, loop_start=0, loop_stop=3, loop_times=2, layers=(
+        L("mamba2", M(heads=3, vdim=13, state=37, groups=3, conv=6, norm_groups=3), 52),
+        L("latent_attention", LA(heads=3, dim=20, vdim=12, kv_rank=34, scale=0.3), None),
+        L("attention", A(heads=3, kv_heads=1, dim=20, vdim=12, scale=0.3, rot=Rot(10, 50000.0, Bands(8.0, 0.5, 2.0, 32.0)), window=70), 41)))
+    # a width that the weight-streaming kernels take, heads of a matrix-core size, one layer looped
+    S = MorulixConfig(vocab=300, width=512, norm_eps=1e-6, loop_start=1, loop_stop=2, loop_times=2, layers=(
+        L("attention", A(heads=8, kv_heads=2, dim=64, vdim=64, scale=0.11, rot=Rot(32, 250000.0, Bands(8.0, 1.0, 4.0, 512.0)), window=130), 640),
+        L("mamba2", M(heads=8, vdim=64, state=128, groups=2, conv=4, norm_groups=4), 640),
+        L("latent_attention", LA(heads=8, dim=64, vdim=64, kv_rank=256, scale=0.1), 640)))
+    # no loop; more heads than a matrix-core tile has rows, state-space heads of more than a workgroup's channels and rows
+    T = MorulixConfig(vocab=160, width=256, norm_eps=1e-5, layers=(
+        L("latent_attention", LA(heads=40, dim=16, vdim=8, kv_rank=512, scale=0.3), 192),
+        L("mamba2", M(heads=4, vdim=80, state=160, groups=2, conv=3, norm_groups=1), 320),
+        L("attention", A(heads=4, kv_heads=1, dim=96, vdim=96, scale=0.1, rot=Rot(96, 20000.0), window=50), 192)))
+    return {"P": (P, 3), "Q": (Q, 4), "R": (R, 5), "S": (S, 6), "T": (T, 7)}
