@@ -45,6 +45,13 @@ input, gated linear attention in turn with windowed attention beside a recurrenc
 feed-forwards with identity experts and a gated shared expert) beside the Bafarax decoder, the closest of the engine's
 models, at equal layer sizes, in the same way. One JSON line.
 
+    python bench.py --morulix [--shape 1b|3b] [--layers L] [--kernels-only]
+
+measures the Morulix decoder (one norm for both sublayers on a 32-bit stream; state-space mixers with one decay per head,
+windowed attention and attention through a latent with learned sinks and a gate per head; a stretch of layers run twice,
+each pass behind a projection of the stream and the embedded tokens) beside the Bafarax decoder, the closest of the
+engine's models, at equal layer sizes and as many runs of a layer, in the same way. One JSON line.
+
     python bench.py --scenario requests-3b | chunked-8b [--layers L]
 
 runs a whole workload through `LLM.generate` instead and prints one JSON line of its own: many
@@ -1026,6 +1033,193 @@ def tegolix(args) -> int:
     return 0
 
 
+def morulix_design(shape: str, layers: int | None):
+    """The Morulix configuration that `--morulix` measures at the layer sizes of `shape`, and those sizes by name."""
+    from tinyserve_llm_amd.config.morulix import (FrequencyBands, MorulixAttention, MorulixConfig, MorulixLatentAttention, MorulixLayer,
+                                                  MorulixMamba2, MorulixRotation)
+    sizes = SHAPES[shape]
+    sh = sizes["shape"]
+    runs = layers or sizes["layers_full"]
+    hidden, nh, nkv, hd, inter, vocab = (sh["hidden_size"], sh["num_attention_heads"], sh["num_key_value_heads"], sh["head_dim"],
+                                         sh["intermediate_size"], sh["vocab_size"])
+    # state-space heads of 64 channels, twice the width of them together, with 128 state rows and 8 groups; a window and a
+    # latent as long and as large as Bafarax's; of the runs of a layer, four are a second pass over four layers
+    window, rank, sv, sn, sg, taps = 1024, 256, 64, 128, 8, 4
+    shd = 2 * hidden // sv
+    att = MorulixAttention(heads=nh, kv_heads=nkv, dim=hd, vdim=hd, scale=hd ** -0.5, window=window,
+                           rot=MorulixRotation(hd // 2, 500000.0, FrequencyBands(factor=8.0, low=1.0, high=4.0, original=8192.0)))
+    lat = MorulixLatentAttention(heads=nh, dim=hd, vdim=hd, kv_rank=rank, scale=hd ** -0.5)
+    ssm = MorulixMamba2(heads=shd, vdim=sv, state=sn, groups=sg, conv=taps, norm_groups=sg)
+    cycle = (("mamba2", ssm), ("attention", att), ("mamba2", ssm), ("latent_attention", lat))
+    looped = runs >= 8
+    own = runs - 4 if looped else runs
+    loop = dict(loop_start=own // 8 * 4, loop_stop=own // 8 * 4 + 4, loop_times=2) if looped else {}
+    mor = MorulixConfig(vocab=vocab, width=hidden, norm_eps=1e-6, layers=tuple(MorulixLayer(*cycle[i % 4], inter) for i in range(own)), **loop)
+    return mor, dict(window=window, rank=rank, ssm_heads=shd, ssm_vdim=sv, ssm_state=sn, ssm_groups=sg, conv_taps=taps, layers=own,
+                     runs=len(mor.run_order()), loop=loop)
+
+
+def morulix(args) -> int:
+    """The Morulix decoder beside the Bafarax decoder (the engine's closest design: a 32-bit stream with norms stored around
+    zero, attention through a latent, a recurrence with a matrix per head) at the layer sizes of `--shape`: whole-engine
+    throughput, and the like kernels of the two side by side. One JSON line."""
+    import torch
+
+    from tinyserve_llm_amd.ops import hip
+    from tinyserve_llm_amd.parts.linear import linear
+
+    baf, z = bafarax_design(args.shape, args.layers)
+    mor, t = morulix_design(args.shape, args.layers)
+    hidden, nh, nkv, hd, vocab = z["hidden"], z["nh"], z["nkv"], z["hd"], z["vocab"]
+    chunk, rot, mh, md, mv = z["chunk"], z["rot"], z["mh"], z["md"], z["mv"]
+    window, rank = t["window"], t["rank"]
+    prompt_len = args.context
+    bench = DesignBench(vocab, prompt_len)
+    timed, context = bench.timed, bench.context
+    bf = torch.bfloat16
+
+    def kernel_pairs() -> dict:
+        pairs = {}
+        pool_page = 32
+        peaks = hip.measure_peaks()
+        read_peak, mfma_peak, vector_peak = peaks["read_GBps"] * 1e9, peaks["mfma_bf16_TFLOPs"] * 1e12, PEAK_FLOPS["fp32"]
+        sinks = torch.randn(nh, device="cuda")
+        sizes = hip.SsdSizes(t["ssm_heads"], t["ssm_vdim"], t["ssm_groups"], t["ssm_state"], t["conv_taps"])
+        for label, starts, counts in (("prompt portion", [0], [prompt_len]), ("decoded tokens, batch 64", [prompt_len + chunk // 2 - 1] * 64, [1] * 64),
+                                      ("decoded token", [prompt_len + chunk // 2 - 1], [1])):
+            ctx, slots, pages = context(starts, counts, pool_page)
+            T, prompt, R = ctx.num_tokens, ctx.num_tokens > 64, len(starts)
+            of_peak = lambda flops, nbytes, us: ({"frac_of_mfma": flops / us * 1e6 / mfma_peak} if prompt else
+                                                 {"frac_of_read": nbytes / us * 1e6 / read_peak})
+            k = torch.randn(pages, nkv, pool_page, hd, device="cuda").to(bf).permute(0, 2, 1, 3)
+            v = torch.randn(pages, nkv, hd, pool_page, device="cuda").to(bf).permute(0, 3, 1, 2)
+            q = torch.randn(T, nh, hd, device="cuda").to(bf)
+            spans = list(zip(starts, counts))
+            seen_w = sum(min(p + 1, window) for s0, n in spans for p in range(s0, s0 + n))
+            seen_c = sum(p % chunk + 1 for s0, n in spans for p in range(s0, s0 + n))
+            seen_a = sum(p + 1 for s0, n in spans for p in range(s0, s0 + n))
+            # attention in a window, against attention in chunks with learned sinks
+            us_m = timed(lambda: hip.paged_attention(q, k, v, ctx, 0, hd ** -0.5, window))
+            us_b = timed(lambda: hip.paged_attention(q, k, v, ctx, 0, hd ** -0.5, 0, sinks=sinks, chunk_mask=chunk))
+            pairs[f"attention, {label}"] = {
+                "morulix_us": us_m, "bafarax_us": us_b, "morulix_keys": seen_w, "bafarax_keys": seen_c,
+                "morulix": of_peak(4 * nh * hd * seen_w, seen_w * 2 * nkv * hd * 2, us_m),
+                "bafarax": of_peak(4 * nh * hd * seen_c, seen_c * 2 * nkv * hd * 2, us_b)}
+            # attention through a latent: every position before, no turned part, a sink and a gate per head in the attention
+            # kernel; against a window, a turned part and a gate per element in the product behind it
+            rec = {}
+            for name, r, seen, win in (("morulix", 0, seen_a, 0), ("bafarax", rot, seen_w, window)):
+                cache = torch.randn(pages, pool_page, 1, rank + r, device="cuda").to(bf)
+                values = cache[:, :, :, :rank].permute(0, 2, 3, 1).contiguous().permute(0, 3, 1, 2)      # transposed inside a page
+                q32 = torch.randn(T, nh, hd + r, device="cuda")
+                uk_t = (torch.randn(nh, rank, hd, device="cuda") * 0.05).to(bf)
+                uv = (torch.randn(nh, hd, rank, device="cuda") * 0.05).to(bf)
+                freqs = torch.rand(rot // 2, dtype=torch.float64, device="cuda")
+                absorbed = torch.empty(T, nh, rank + r, device="cuda")
+                heads = torch.empty(T, nh, hd, dtype=bf, device="cuda")
+                wide, per_head = torch.randn(T, nh * hd, device="cuda"), torch.randn(T, nh, device="cuda")
+                extra = dict(sinks=sinks, head_gate=per_head) if r == 0 else {}
+
+                def before():
+                    hip.heads_gemm(q32[:, :, :hd], uk_t.transpose(1, 2), absorbed[:, :, :rank])
+                    if r:
+                        hip.rotate_heads(absorbed[:, :, rank:], q32[:, :, hd:], freqs, 1.2, ctx.positions, interleaved=True)
+                before()
+                attend = lambda: hip.paged_attention_latent(absorbed, cache, rank, ctx, 0, (hd + r) ** -0.5, win, 0, out_dtype=bf, v_cache=values, **extra)
+                mixed = attend()
+                us_before, us_att = timed(before), timed(attend)
+                us_after = timed(lambda: hip.heads_gemm(mixed, uv.transpose(1, 2), heads, gate=wide if r else None))
+                rec.update({f"{name}_attention_us": us_att, f"{name}_before_us": us_before, f"{name}_after_us": us_after, f"{name}_keys": seen,
+                            name + "_attention": of_peak(2 * nh * seen * (2 * rank + r), seen * (2 * rank + r) * 2, us_att),
+                            name + "_products": of_peak(4 * T * nh * hd * rank, 4 * nh * hd * rank * 2 + T * nh * (2 * rank + r) * 4, us_before + us_after)})
+            pairs[f"attention through a latent, {label}"] = rec
+            # between projection and cache
+            qkv_row = (nh + 2 * nkv) * hd
+            qkv32 = torch.randn(T, qkv_row, device="cuda")
+            qw, kw = torch.ones(nh * hd, device="cuda"), torch.ones(nkv * hd, device="cuda")
+            rfreqs, hfreqs = torch.rand(hd // 2, dtype=torch.float64, device="cuda"), torch.rand(hd // 4, dtype=torch.float64, device="cuda")
+
+            def baf_finish():
+                hip.segment_rmsnorm_pair(qkv32, (0, nh * hd, qw), (nh * hd, nkv * hd, kw), 1e-6)
+                return hip.qkv_finish(qkv32, rfreqs, ctx.positions, slots, k, v, nh, nkv, hd, hd, bf, interleaved=False)
+            us_m = timed(lambda: hip.qkv_finish(qkv32, hfreqs, ctx.positions, slots, k, v, nh, nkv, hd, hd, bf, interleaved=False))
+            us_b = timed(baf_finish)
+            mbytes, bbytes = T * qkv_row * (4 + 2), T * qkv_row * (4 + 4 + 4 + 2)
+            down = torch.randn(T, nh * hd + rank + nh, device="cuda")
+            lcache = torch.zeros(pages, pool_page, 1, rank, device="cuda", dtype=bf)
+            lvalues = torch.zeros(pages, 1, rank, pool_page, device="cuda", dtype=bf).permute(0, 3, 1, 2)
+            lcw = torch.ones(rank, device="cuda")
+            us_l = timed(lambda: hip.latent_finish(down, 0, 0, nh * hd, rank, 0, None, lcw, 1e-6, None, 1.0, ctx.positions, slots, lcache, bf, v_cache=lvalues))
+            lbytes = T * rank * (4 + 2 + 2)
+            pairs[f"between projection and cache, {label}"] = {
+                "morulix_us": us_m, "morulix_latent_us": us_l, "bafarax_us": us_b, "morulix_bytes": mbytes, "bafarax_bytes": bbytes,
+                "morulix_frac_of_read": mbytes / us_m * 1e6 / read_peak, "morulix_latent_frac_of_read": lbytes / us_l * 1e6 / read_peak,
+                "bafarax_frac_of_read": bbytes / us_b * 1e6 / read_peak}
+            # the stream's sum and the norm that reads it: two branches once a layer, against one twice a layer
+            x32, a32, b32 = (torch.randn(T, hidden, device="cuda") for _ in range(3))
+            w32 = torch.ones(hidden, device="cuda")
+            us_m = timed(lambda: hip.stream_update_norm(x32, a32, b32, None, 1.0, (w32, None), 1e-6, out_dtype=bf))
+            us_b = timed(lambda: hip.stream_update_norm(x32, a32, None, None, 1.0, (w32, None), 1e-6, out_dtype=bf))
+            mbytes, bbytes = T * hidden * (4 * 4 + 2), T * hidden * (3 * 4 + 2)
+            pairs[f"stream sum and norm, {label}"] = {"morulix_us": us_m, "bafarax_us": us_b, "morulix_bytes": mbytes, "bafarax_bytes": bbytes,
+                                                      "morulix_frac_of_read": mbytes / us_m * 1e6 / read_peak,
+                                                      "bafarax_frac_of_read": bbytes / us_b * 1e6 / read_peak}
+            # the input of a pass (operand, then product), against a product of the same size alone
+            w_in = (torch.randn(hidden, 2 * hidden, device="cuda") * 0.02).to(bf)
+            us_join = timed(lambda: hip.stream_join(x32, a32, b32, x32, bf))
+            joined = hip.stream_join(x32, a32, b32, x32, bf)
+            us_in = timed(lambda: linear(joined, w_in, out_dtype=torch.float32))
+            jbytes = T * hidden * (4 * 4 + 2 * 2)
+            pairs[f"input of a pass, {label}"] = {"operand_us": us_join, "operand_bytes": jbytes, "operand_frac_of_read": jbytes / us_join * 1e6 / read_peak,
+                                                  "product_us": us_in, "product": of_peak(4 * T * hidden * hidden, 2 * hidden * hidden * 2, us_in)}
+            # the recurrences: convolution and step sizes, scan, gated norm; against the matrix memory's scan and norm
+            proj = torch.randn(T, -(-sizes.projected // 8) * 8, device="cuda")
+            conv, cbias = torch.randn(sizes.taps, sizes.row, device="cuda") * 0.4, torch.zeros(sizes.row, device="cuda")
+            dtb, alog, skip = torch.full((sizes.heads,), -3.0, device="cuda"), torch.zeros(sizes.heads, device="cuda"), torch.ones(sizes.heads, device="cuda")
+            nw = torch.ones(sizes.inner, device="cuda")
+            state = torch.zeros(R, sizes.matrix + sizes.kept, device="cuda")
+            prepare = lambda: hip.ssd_prepare(proj, conv, cbias, dtb, alog, state, ctx, sizes, bf)
+            mixed, steps, logs = prepare()
+            y = hip.ssd_scan(mixed, steps, logs, skip, state, ctx, sizes)
+            us_p, us_s = timed(prepare), timed(lambda: hip.ssd_scan(mixed, steps, logs, skip, state, ctx, sizes))
+            us_n = timed(lambda: hip.gated_group_norm(y, proj[:, :sizes.inner], nw, t["ssm_groups"], 1e-6, bf))
+            pbytes = T * (sizes.channels * (4 + 2) + sizes.heads * 12) + 2 * R * sizes.kept * 4
+            sbytes = T * (sizes.row * 2 + sizes.heads * 8 + sizes.inner * 4) + 2 * R * sizes.matrix * 4
+            nbytes = T * sizes.inner * (4 + 4 + 2)
+            sflops = 4 * T * sizes.heads * sizes.vdim * sizes.state
+            width = 2 * mh * md + mh * mv + 2 * mh + mh * mv
+            mproj = torch.randn(T, width, device="cuda")
+            gb, mw = torch.zeros(2 * mh, device="cuda"), torch.ones(mh * mv, device="cuda")
+            mstate = torch.zeros(R, hip.mlstm_state_size(mh, md, mv), device="cuda")
+            scan_b = lambda: hip.mlstm_scan(mproj, gb[:mh], gb[mh:], mstate, ctx.cu_seqlens, ctx.state_slots, mh, md, mv, 15.0,
+                                            host_cu_seqlens=ctx.host_cu_seqlens, scratch=ctx.scratch)
+            o = scan_b()
+            us_b = timed(scan_b)
+            us_bn = timed(lambda: hip.mlstm_finish(o, mw, mproj[:, width - mh * mv:], mh, mv, 1e-6, bf))
+            bbytes = T * ((width - mh * mv) * 4 + mh * mv * 4) + 2 * R * mstate.shape[1] * 4
+            bnbytes = T * mh * mv * (4 + 4 + 2)
+            bflops = 4 * T * mh * md * mv
+            pairs[f"recurrence, {label}"] = {
+                "morulix_convolution_us": us_p, "morulix_scan_us": us_s, "morulix_norm_us": us_n, "bafarax_scan_us": us_b, "bafarax_norm_us": us_bn,
+                "morulix_scan_bytes": sbytes, "bafarax_scan_bytes": bbytes, "morulix_flops": sflops, "bafarax_flops": bflops,
+                "morulix_convolution_frac_of_read": pbytes / us_p * 1e6 / read_peak, "morulix_scan_frac_of_read": sbytes / us_s * 1e6 / read_peak,
+                "morulix_norm_frac_of_read": nbytes / us_n * 1e6 / read_peak, "bafarax_scan_frac_of_read": bbytes / us_b * 1e6 / read_peak,
+                "bafarax_norm_frac_of_read": bnbytes / us_bn * 1e6 / read_peak,
+                "morulix_scan_frac_of_fp32_vector": sflops / us_s * 1e6 / vector_peak, "bafarax_scan_frac_of_fp32_vector": bflops / us_b * 1e6 / vector_peak}
+        pairs["peaks"] = {"read_GBps": read_peak / 1e9, "mfma_bf16_TFLOPs": mfma_peak / 1e12, "fp32_vector_TFLOPs_published": vector_peak / 1e12}
+        return pairs
+
+    record = {"designs": {} if args.kernels_only else {"bafarax": bench.whole_engine(baf), "morulix": bench.whole_engine(mor)},
+              "kernels": kernel_pairs(),
+              "config": {"shape": args.shape, "hidden": hidden, "heads": nh, "kv_heads": nkv, "head_dim": hd, "bafarax_layers": z["layers"], "morulix": t,
+                         "morulix_layers": "in turn: a state-space mixer, windowed attention, a state-space mixer, attention through a latent, all with "
+                                           "a dense feed-forward of the shape's width",
+                         "bafarax_memory": {"heads": mh, "dim": md, "vdim": mv}, "bafarax_chunk": chunk, "bafarax_window": z["window"],
+                         "vocab": vocab, "context": prompt_len, "dtype": "bf16", "data": "synthetic uniform token ids, random weights"}}
+    print(json.dumps(record))
+    return 0
+
+
 def kernel_classes(llm, config, batch: int, reps: int = 5) -> dict:
     """Times one decode step's kernels by class. An eager step (no graph) is run once with every
     launch of the engine's kernel module noted down with its operands; then each class's launches
@@ -1161,7 +1355,9 @@ def main() -> int:
                          "throughput and the like kernels side by side; one JSON line")
     ap.add_argument("--tegolix", action="store_true",
                     help="the Tegolix decoder beside the Bafarax decoder at the layer sizes of --shape: throughput and like kernels")
-    ap.add_argument("--kernels-only", action="store_true", help="with --bafarax or --tegolix: the kernels side by side, no whole-engine runs")
+    ap.add_argument("--morulix", action="store_true",
+                    help="the Morulix decoder beside the Bafarax decoder at the layer sizes of --shape: throughput and like kernels")
+    ap.add_argument("--kernels-only", action="store_true", help="with --bafarax, --tegolix or --morulix: the kernels side by side, no whole-engine runs")
     ap.add_argument("--kernel-classes", action="store_true",
                     help="time one decode step's kernels class by class (bytes, microseconds, GB/s) and exit")
     ap.add_argument("--peaks", action="store_true",
@@ -1193,6 +1389,8 @@ def main() -> int:
         return bafarax(args)
     if args.tegolix:
         return tegolix(args)
+    if args.morulix:
+        return morulix(args)
     sizes = SHAPES[args.shape]
     full_layers = sizes["layers_full"]
     args.layers = args.layers or full_layers

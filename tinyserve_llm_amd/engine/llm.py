@@ -6,6 +6,7 @@ one, the next is already scheduled and packed (see `LLM.step`)."""
 from __future__ import annotations
 
 import logging
+import math
 import os
 import time
 from dataclasses import dataclass, replace
@@ -142,14 +143,15 @@ class LLM:
     def _size_from_free_memory(self, sc: SchedulerConfig, cc: CacheConfig, utilisation: float, graph_memory: int) -> int:
         """Pages from what the GPU has left under the utilisation limit, after setting aside what is
         allocated later: the activations of a worst-case step (llm_engine.py:112-140 measures them
-        with a trial step; here the parts say how wide they get), the matrix library's workspace and
-        the buffer its timing sweeps, and the recorded decode steps' own buffers (`graph_memory`,
+        with a trial step; here the parts say how wide they get), the requests' state slots, the matrix
+        library's workspace and the buffer its timing sweeps, and the recorded decode steps' own buffers (`graph_memory`,
         which `DecodeGraphs` holds itself to)."""
         from tinyserve_llm_amd.ops import hip
         free, total = torch.cuda.mem_get_info(self.device)
         widest = self.model.widest_activation()
         act = sc.max_num_batched_tokens * widest * 4 * 6 + sc.max_num_seqs * self.model.spec.vocab_size * 4 * 2
-        later = act + graph_memory + hip.LIBRARY_WORKSPACE_BYTES + hip.LIBRARY_TUNING_SWEEP_BYTES
+        states = sc.max_num_seqs * sum(math.prod(e.state.shape) * e.state.dtype.itemsize for e in self.model.state_plan())
+        later = act + states + graph_memory + hip.LIBRARY_WORKSPACE_BYTES + hip.LIBRARY_TUNING_SWEEP_BYTES
         budget = total * utilisation - (total - free) - later
         per_page = max(1, bytes_per_page(self.model, cc.block_size, self.dtype))
         pages = int(budget // per_page)
