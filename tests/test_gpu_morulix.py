@@ -360,6 +360,32 @@ def test_recurrence_over_steps_and_slots(dtype, kind, portions, slow):
     assert torch.equal(state[[1, 3]], before[[1, 3]]) and torch.equal(state[:, z.matrix:], before[:, z.matrix:])
 
 
+@pytest.mark.parametrize("portions", ["whole", "two"])
+@pytest.mark.parametrize("dtype", DTYPES)
+def test_tokens_that_forget_everything_between_tokens_that_forget_nothing(dtype, portions):
+    """Log decays of -1e-4 beside ones of -30, -3,000 and -1e30: what lies between two forgetful tokens is carried as
+    precisely as ever, and a forgetful token leaves nothing behind (and no NaN)."""
+    h = hip()
+    z, W, dev, gen = ssd_setup("plain", dtype)
+    n = 280
+    m, d, _, _ = scan_inputs("plain", dtype, [n], gen, z, True)[0]
+    logs = torch.full((n, z.heads), -1e-4)
+    for t, l in ((10, -3000.0), (11, -3000.0), (40, -30.0), (63, -3000.0), (64, -1e30), (100, -1e30), (101, -3000.0), (200, -1.0), (255, -1e30)):
+        logs[t] = l
+    state, out = torch.zeros(1, z.matrix + z.kept, device=DEV), []
+    for step, ctx in packed_steps([n], PORTIONS[portions], [0]):
+        (_, a, k), = step
+        out.append(h.ssd_scan(m[a:a + k].to(DEV), d[a:a + k].to(DEV), logs[a:a + k].to(DEV), dev["skip"], state, ctx, z))
+    got = torch.cat(out).cpu().to(F64)
+    S, want = torch.zeros(z.heads, z.state, z.vdim, dtype=F64), []
+    for t in range(n):                                       # (a rate per token that makes exp(-rate d) the decay it is to have)
+        y, S = plain_scan(z, m[t:t + 1], d[t:t + 1], -(logs[t].to(F64) / d[t].to(F64)), dev["skip"].cpu(), S)
+        want.append(y.reshape(-1))
+    want = torch.stack(want)
+    size = max(1.0, float(want.abs().max()))
+    torch.testing.assert_close(got, want, atol=3e-5 * size, rtol=3e-5)
+
+
 @pytest.mark.parametrize("dtype", DTYPES)
 def test_a_token_is_read_out_hundreds_of_tokens_later(dtype):
     """One token writes to rows of the state that no other token writes to, and one far later query reads only those rows:

@@ -330,12 +330,14 @@ extern "C" int ts_ssd_step(float* out, const void* mixed, int dtype, const float
 // ---- chunks of 64 tokens on the matrix cores (bfloat16) ----------------------------------------------------------
 
 // In the first wave, lane t: the running sum of the log decays up to token t of the chunk (tokens past its end add 0).
-static __device__ __forceinline__ float ss_running(const float* __restrict__ logs, int tok0, int len, int heads, int h) {
+// Differences of two such sums are what counts, and one token may decay by thousands where its neighbours hardly do: the
+// sums are 64-bit. A log decay below -128 counts as -128 (its exponential is 0 in 32-bit either way).
+static __device__ __forceinline__ double ss_running(const float* __restrict__ logs, int tok0, int len, int heads, int h) {
   const int t = threadIdx.x;
-  float b = t < len ? logs[(int64_t)(tok0 + t) * heads + h] : 0.f;
+  double b = t < len ? (double)fmaxf(logs[(int64_t)(tok0 + t) * heads + h], -128.f) : 0.0;
 #pragma unroll
   for (int off = 1; off < TS_WAVE; off <<= 1) {
-    const float up = __shfl_up(b, off, TS_WAVE);
+    const double up = __shfl_up(b, off, TS_WAVE);
     if (t >= off) b += up;
   }
   return b;
@@ -387,10 +389,10 @@ ssd_chunk_sums_kernel(float* __restrict__ buf, float* __restrict__ totals, const
   const int row = heads * vp + 2 * groups * np, g = h / (heads / groups);
   const int wave = wave_index(), lane = threadIdx.x & (TS_WAVE - 1), r = lane & 15, q = lane >> 4;
   if (threadIdx.x < TS_WAVE) {
-    const float b = ss_running(logs, tok0, len, heads, h);
-    const float total = __shfl(b, TS_WAVE - 1, TS_WAVE);
-    weight_s[lane] = lane < len ? expf(total - b) * steps[(int64_t)(tok0 + lane) * heads + h] : 0.f;
-    if (lane == 0 && blockIdx.z == 0) totals[(int64_t)chunk * heads + h] = total;
+    const double b = ss_running(logs, tok0, len, heads, h);
+    const double total = __shfl(b, TS_WAVE - 1, TS_WAVE);
+    weight_s[lane] = lane < len ? expf((float)(total - b)) * steps[(int64_t)(tok0 + lane) * heads + h] : 0.f;
+    if (lane == 0 && blockIdx.z == 0) totals[(int64_t)chunk * heads + h] = (float)total;
   }
   __syncthreads();
   ss_turn<true>(x_s, xr_s, mixed + h * vp + v0, row, tok0, len, vp - v0, weight_s);
@@ -472,7 +474,8 @@ ssd_chunk_out_kernel(float* __restrict__ out, const float* __restrict__ buf, con
   constexpr int np = 32 * NQ;
   __shared__ __attribute__((aligned(16))) bf16_t x_s[64][SS_PAD];                      // x, turned: [channel][token]
   __shared__ __attribute__((aligned(16))) bf16_t p_s[SS_L][SS_PAD], pr_s[SS_L][SS_PAD];  // weights: [token][key token], two terms
-  __shared__ float b_s[SS_L], d_s[SS_L];
+  __shared__ double b_s[SS_L];
+  __shared__ float d_s[SS_L];
   const int chunk = blockIdx.x, h = blockIdx.y, v0 = blockIdx.z * 64;
   const int tok0 = chunks[4 * chunk], len = chunks[4 * chunk + 1];
   const int row = heads * vp + 2 * groups * np, g = h / (heads / groups);
@@ -519,7 +522,7 @@ ssd_chunk_out_kernel(float* __restrict__ out, const float* __restrict__ buf, con
         for (int k = 0; k < 2; ++k) {
           const int e = 2 * j + k, key = 32 * kk + 8 * q + e;
           const float s = st[kk][e >> 2][e & 3];
-          p[k] = (key <= t && t < len) ? s * expf(b_s[t] - b_s[key]) * d_s[key] : 0.f;
+          p[k] = (key <= t && t < len) ? s * expf((float)(b_s[t] - b_s[key])) * d_s[key] : 0.f;
         }
         (&hi.x)[j] = pack_bf16(p[0], p[1]);
         (&lo.x)[j] = ss_rest((&hi.x)[j], p[0], p[1]);
@@ -558,7 +561,7 @@ ssd_chunk_out_kernel(float* __restrict__ out, const float* __restrict__ buf, con
 #pragma unroll
   for (int tb = 0; tb < 4; ++tb) {
     const int tok = 16 * tb + r;
-    const float decay = expf(b_s[tok]);
+    const float decay = expf((float)b_s[tok]);
 #pragma unroll
     for (int j = 0; j < 4; ++j) acc[tb][j] *= decay;
 #pragma unroll
