@@ -396,7 +396,7 @@ def test_softmax_over_all_outputs_identity_experts_and_a_gated_shared_expert(dty
 def test_relu_gated_unit():
     h = hip()
     sums = torch.randn(6, 2 * 37) * 2
-    got = h.capped_glu(sums.to(DEV), 0.0, 1.0, 0.0, torch.float32, relu=True)
+    got = h.capped_glu(sums.to(DEV), 0.0, 1.0, 0.0, torch.float32, activation="relu")
     torch.testing.assert_close(got.cpu(), torch.relu(sums[:, :37]) * sums[:, 37:], atol=1e-6, rtol=1e-6)
 
 

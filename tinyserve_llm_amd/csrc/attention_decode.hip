@@ -131,7 +131,7 @@ attn_decode_mfma_kernel(bf16_t* __restrict__ out, float* __restrict__ part_o, fl
     if (num_splits == 1) {                  // the whole context was this workgroup's: position `pos` is always visible
       if (GENERAL && sink) L += fast_exp2((sinks ? sinks[kvh * G + head] * 1.44269504088896340736f : 0.f) - M);
       float y = acc / L;
-      if (GENERAL) y *= ts_out_gate(gate, (int64_t)t * gate_stride + ((int64_t)kvh * G + head) * HD + d);
+      if (GENERAL) y *= ts_out_gate(gate, gate_stride, t, kvh * G + head, HD, d);
       out[((int64_t)t * nh + (int64_t)kvh * G + head) * HD + d] = f2bf(y);
     } else {
       const int64_t row = ((int64_t)t * nh + (int64_t)kvh * G + head) * num_splits + split;
@@ -177,7 +177,7 @@ attn_decode_combine_kernel(bf16_t* __restrict__ out, const float* __restrict__ p
     float acc = 0.f;
 #pragma unroll 4
     for (int s = 0; s <= s1 - s0; ++s) acc = fmaf(po[(int64_t)s * hd + d], wgt[s], acc);
-    out[th * hd + d] = f2bf(acc * inv * ts_out_gate(gate, (int64_t)t * gate_stride + (int64_t)(blockIdx.x % nh) * hd + d));
+    out[th * hd + d] = f2bf(acc * inv * ts_out_gate(gate, gate_stride, t, blockIdx.x % nh, hd, d));
   }
 }
 
@@ -216,7 +216,7 @@ static int launch_decode(void* out, float* part_o, float* part_ml, const void* q
                          int waves, float scale, int window, int page_run, int combine, bool general, float softcap, int sink,
                          const float* sinks, const float* slopes, const float* gate, int64_t gate_stride, hipStream_t stream) {
   if (num_tokens <= 0) return TS_OK;
-  if (gate && (!general || !combine || gate_stride < (int64_t)nh * hd)) return TS_BAD_SHAPE;
+  if (gate && (!general || !combine || (gate_stride < (int64_t)nh * hd && -gate_stride < nh))) return TS_BAD_SHAPE;
   if (nkv <= 0 || nh % nkv || page_size <= 0 || page_size % 8 || max_blocks <= 0 || num_splits <= 0 || page_run < 0 || page_run > 16)
     return TS_BAD_SHAPE;
   if (waves < 1 || waves > DEC_WAVES_FOR(hd, chunk == 32 * waves) || chunk <= 0 || chunk % (32 * waves) || num_splits > COMBINE_MAX_SPLITS)
@@ -279,7 +279,8 @@ extern "C" int ts_paged_attention_decode(void* out, float* part_o, float* part_m
 // The same with capped scores (softcap > 0: cap * tanh(score / cap)), a sink (one more in the softmax's
 // denominator; `sinks`, float [nh], if given: exp(sinks[head]) more instead), a penalty of slopes[head] (float [nh],
 // if given) per position of distance taken off every score, and weights carried in two bfloat16 terms; always combines.
-// `gate` (float [tokens, >= nh hd], rows gate_stride apart; may be null): the output leaves multiplied by sigmoid(gate).
+// `gate` (float [tokens, >= nh hd], rows gate_stride apart; may be null): the output leaves multiplied by sigmoid(gate);
+// a stride below zero: one number per head (`ts_out_gate`).
 extern "C" int ts_paged_attention_decode_general(void* out, float* part_o, float* part_ml, const void* q, const void* k_cache,
                                                  const void* v_cache, const int32_t* block_tables,
                                                  const int32_t* seq_of_token, const int32_t* positions, int num_tokens,

@@ -11,7 +11,7 @@
 //     optionally with a sink: a key of score 0 that has no value, i.e. one more in the denominator; or with
 //     learned sinks, exp(sinks[head]) in the denominator instead of 1. Optionally a penalty on distance,
 //     slopes[head] * (position - key's position), is taken off every score, and the output row is multiplied
-//     element by element by sigmoid(gate) on its way out (gate: 32-bit rows of the step, one element per output).
+//     element by element by sigmoid(gate) on its way out (gate: 32-bit rows of the step, one element per output, or, with a stride below zero, one per head).
 //     Scores, weights and the weighted sum are 32-bit. Keys are visited in chunks of 64 counted from position
 //     0, so the order of every sum depends on the token's position alone.
 #include "common.h"
@@ -19,6 +19,7 @@
 #define AG_WAVES 4
 #define AG_MAX_HD 256
 
+// row: elements from one token's projected row q | k | v to the next (columns behind them are not read).
 // One workgroup per token: the token's angles are taken once (sine and cosine of position * f_i for every pair,
 // left in LDS), then the workgroup's waves take the token's heads in turn, one head a wave at a time.
 template <typename TI, typename TO>
@@ -27,7 +28,7 @@ qkv_finish_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* __restri
                   const double* __restrict__ freqs, const int32_t* __restrict__ positions,
                   const int32_t* __restrict__ slots, int num_tokens, int nh, int nkv, int hd, int vd_size, int rot,
                   int interleaved, int qk_norm, float qk_eps, int v_norm, float v_eps, int page_size, int64_t kp,
-                  int64_t ks, int64_t kh, int64_t vp, int64_t vs, int64_t vh, int64_t vd, int with_values, float amplitude) {
+                  int64_t ks, int64_t kh, int64_t vp, int64_t vs, int64_t vh, int64_t vd, int with_values, float amplitude, int64_t row) {
   __shared__ float head_s[AG_WAVES][AG_MAX_HD];
   __shared__ float cos_s[AG_MAX_HD / 2], sin_s[AG_MAX_HD / 2];
   const int wave = threadIdx.x / TS_WAVE, lane = threadIdx.x & (TS_WAVE - 1);
@@ -46,7 +47,6 @@ qkv_finish_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* __restri
     sin_s[pair] = sn * amplitude;
   }
   __syncthreads();
-  const int64_t row = (int64_t)(nh + nkv) * hd + (int64_t)nkv * vd_size;
   const int slot = slots ? slots[t] : -1;
   const bool stores = slot >= 0 && k_cache;
   const int page = stores ? slot / page_size : 0, off = stores ? slot - page * page_size : 0;
@@ -132,7 +132,7 @@ qkv_finish_pieces_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* _
                          const double* __restrict__ freqs, const int32_t* __restrict__ positions,
                          const int32_t* __restrict__ slots, int num_tokens, int nh, int nkv, int hd, int vd_size, int rot,
                          int interleaved, int qk_norm, float qk_eps, int v_norm, float v_eps, int page_size, int64_t kp,
-                         int64_t ks, int64_t kh, int64_t vp, int64_t vs, int64_t vh, int64_t vd, int with_values, float amplitude, int slices) {
+                         int64_t ks, int64_t kh, int64_t vp, int64_t vs, int64_t vh, int64_t vd, int with_values, float amplitude, int64_t row, int slices) {
   const int64_t gid = (int64_t)blockIdx.x * (AG_WAVES * TS_WAVE) + threadIdx.x;
   const int piece = (int)(gid % GS);
   const int slice = (int)((gid / GS) % slices);
@@ -163,7 +163,6 @@ qkv_finish_pieces_kernel(TO* __restrict__ q_out, TO* __restrict__ k_cache, TO* _
       if (interleaved && (e & 1)) { cs[e] = cs[e - 1]; sn[e] = sn[e - 1]; }
     }
   };
-  const int64_t row = (int64_t)(nh + nkv) * hd + (int64_t)nkv * vd_size;
   const TI* trow = qkv + (int64_t)t * row;
   // where a head's piece lies in the token's row, and how many of its elements there are for this thread (8 or 0)
   auto piece_of = [&](int h) {
@@ -280,7 +279,7 @@ extern "C" int ts_qkv_finish(void* q_out, void* k_cache, void* v_cache, const vo
                              const int32_t* positions, const int32_t* slots, int num_tokens, int nh, int nkv, int hd,
                              int vd_size, int rot, int interleaved, int qk_norm, float qk_eps, int v_norm, float v_eps,
                              int page_size, int64_t kp, int64_t ks, int64_t kh, int64_t vp, int64_t vs, int64_t vh,
-                             int64_t vd, int in_dtype, int out_dtype, float amplitude, hipStream_t stream) {
+                             int64_t vd, int in_dtype, int out_dtype, float amplitude, int64_t row, hipStream_t stream) {
   if (num_tokens <= 0) return TS_OK;
   if (hd <= 0 || hd > AG_MAX_HD || vd_size <= 0 || vd_size > AG_MAX_HD || nh <= 0 || nkv <= 0 || rot < 0 || rot > hd || rot % 2 ||
       page_size <= 0 || (rot > 0 && !freqs))
@@ -288,11 +287,11 @@ extern "C" int ts_qkv_finish(void* q_out, void* k_cache, void* v_cache, const vo
   // several tokens of a step: their values leave through the tile kernel (a single token's, with its head)
   const int v_tiles = k_cache && num_tokens >= 256 && nkv <= 65535;
   const int64_t blocks = num_tokens;
-  const int64_t row = (int64_t)(nh + nkv) * hd + (int64_t)nkv * vd_size;
+  if (row < (int64_t)(nh + nkv) * hd + (int64_t)nkv * vd_size) return TS_BAD_SHAPE;
   dim3 v_grid((num_tokens + AG_VTOK - 1) / AG_VTOK, nkv);
   // heads in pieces of eight elements: sizes that are multiples of 8 (of 16 where halves are paired), 16-byte aligned rows
   const int in_piece = in_dtype == 0 ? 32 : 16, out_piece = out_dtype == 0 ? 32 : 16;
-  const bool pieces = hd % 8 == 0 && vd_size % 8 == 0 && (interleaved ? rot % 2 == 0 : rot % 16 == 0) &&
+  const bool pieces = hd % 8 == 0 && vd_size % 8 == 0 && row % 8 == 0 && (interleaved ? rot % 2 == 0 : rot % 16 == 0) &&
                       ((uintptr_t)qkv % in_piece) == 0 && ((uintptr_t)q_out % out_piece) == 0 &&
                       (!k_cache || (((uintptr_t)k_cache % out_piece) == 0 && kp % 8 == 0 && ks % 8 == 0 && kh % 8 == 0));
   int gs = 4;
@@ -303,7 +302,7 @@ extern "C" int ts_qkv_finish(void* q_out, void* k_cache, void* v_cache, const vo
   const unsigned piece_blocks = (unsigned)((piece_threads + AG_WAVES * TS_WAVE - 1) / (AG_WAVES * TS_WAVE));
 #define QF_ARGS(TI, TO) \
       (TO*)q_out, (TO*)k_cache, (TO*)v_cache, (const TI*)qkv, freqs, positions, slots, num_tokens, nh, nkv, hd, vd_size, rot, \
-      interleaved, qk_norm, qk_eps, v_norm, v_eps, page_size, kp, ks, kh, vp, vs, vh, vd, !v_tiles, amplitude
+      interleaved, qk_norm, qk_eps, v_norm, v_eps, page_size, kp, ks, kh, vp, vs, vh, vd, !v_tiles, amplitude, row
 #define QF_LAUNCH(TI, TO) \
   if (!pieces) qkv_finish_kernel<TI, TO><<<(unsigned)blocks, AG_WAVES * TS_WAVE, 0, stream>>>(QF_ARGS(TI, TO)); \
   else if (gs == 4) qkv_finish_pieces_kernel<TI, TO, 4><<<piece_blocks, AG_WAVES * TS_WAVE, 0, stream>>>(QF_ARGS(TI, TO), slices); \
@@ -396,7 +395,7 @@ paged_attention_general_kernel(T* __restrict__ out, const T* __restrict__ q, con
     const int d = lane + i * TS_WAVE;
     if (d < vd_size) {
       float o = acc[i] * inv;
-      if (gate) o = o / (1.0f + expf(-gate[(int64_t)t * gate_stride + (int64_t)h * vd_size + d]));
+      if (gate) o = o / (1.0f + expf(-gate[gate_stride >= 0 ? t * gate_stride + (int64_t)h * vd_size + d : h - t * gate_stride]));
       Num<T>::st(orow + d, o);
     }
   }

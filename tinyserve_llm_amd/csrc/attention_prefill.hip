@@ -316,7 +316,7 @@ prefill_tile(PrefillLds<HD>& lds, int tile, int kvh, bf16_t* __restrict__ out, c
 #pragma unroll
         for (int db = 0; db < NDB; ++db) {
           float y = o[j][db][i] * inv;
-          if (GENERAL) y *= ts_out_gate(gate, (int64_t)(t0 + rtk) * gate_stride + ((int64_t)kvh * G + rhh) * HD + 16 * db + r);
+          if (GENERAL) y *= ts_out_gate(gate, gate_stride, t0 + rtk, kvh * G + rhh, HD, 16 * db + r);
           orow[16 * db + r] = f2bf(y);
         }
       }
@@ -363,7 +363,7 @@ static int launch_prefill(void* out, const void* q, const void* k_cache, const v
                           int chunk, float* part_o, float* part_ml, int page_run, bool general, float softcap, int sink,
                           const float* sinks, const float* slopes, const float* gate, int64_t gate_stride, hipStream_t stream) {
   if (num_tiles <= 0) return TS_OK;
-  if (gate && (!general || gate_stride < (int64_t)nh * hd)) return TS_BAD_SHAPE;
+  if (gate && (!general || (gate_stride < (int64_t)nh * hd && -gate_stride < nh))) return TS_BAD_SHAPE;
   if (general && (page_size % 32 || softcap < 0.f)) return TS_BAD_SHAPE;     // (the general variant walks whole steps only)
   const float log2e = 1.44269504088896340736f;
   const float cap_in = softcap > 0.f ? scale / softcap : 0.f, cap_out = softcap * log2e;
@@ -429,7 +429,7 @@ static int launch_prefill(void* out, const void* q, const void* k_cache, const v
   return ts_launch_attention_combine((bf16_t*)out + skip * hd, part_o + skip * num_splits * hd,
                                      part_ml + skip * num_splits * 2, positions + first_token,
                                      num_tokens - first_token, nh, hd, num_splits, chunk, window, stream, general ? sink : 0,
-                                     general ? sinks : nullptr, gate ? gate + (int64_t)first_token * gate_stride : nullptr,
+                                     general ? sinks : nullptr, gate ? gate + (int64_t)first_token * (gate_stride < 0 ? -gate_stride : gate_stride) : nullptr,
                                      gate_stride);
 }
 
@@ -449,7 +449,7 @@ extern "C" int ts_paged_attention_prefill(void* out, const void* q, const void* 
 // denominator; `sinks`, float [nh], if given: exp(sinks[head]) more instead), a penalty of slopes[head] (float [nh],
 // if given) per position of distance taken off every score, and weights carried in two bfloat16 terms; pages of a
 // multiple of 32 keys. `gate` (float [tokens, >= nh hd], rows gate_stride apart; may be null): the output leaves
-// multiplied by sigmoid(gate).
+// multiplied by sigmoid(gate); a stride below zero: one number per head (`ts_out_gate`).
 extern "C" int ts_paged_attention_prefill_general(void* out, const void* q, const void* k_cache, const void* v_cache,
                                                   const int32_t* block_tables, const int32_t* seq_of_token,
                                                   const int32_t* positions, const int32_t* tiles, int num_tiles,

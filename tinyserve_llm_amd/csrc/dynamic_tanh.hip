@@ -164,12 +164,19 @@ extern "C" int ts_embedding_dyt_stream(float* out, const void* table, int dtype,
   return ts_check_launch();
 }
 
+// What the gate passes: 0 g sigmoid(slope g), 1 relu, 2 gelu in its tanh form.
+static __device__ __forceinline__ float dt_gate(float g, float slope, int act) {
+  if (act == 1) return fmaxf(g, 0.f);
+  if (act == 2) return 0.5f * g * (1.0f + tanhf(0.7978845608028654f * (g + 0.044715f * g * g * g)));
+  return g / (1.0f + expf(-slope * g));
+}
+
 // The capped gated unit between the two projections of a feed-forward: from a row [gate | up] of 32-bit (or
-// stored) sums, g = min(gate, limit), u = clamp(up, -limit, limit), y = g sigmoid(slope g) (u + 1).
-// limit <= 0: no cap. Rows may be picked through `row_stride` (a row of the operand may be wider than 2 ff).
+// stored) sums, g = min(gate, limit), u = clamp(up, -limit, limit), y = act(g) (u + up_shift) with act(g) = g sigmoid(slope g) (act 0),
+// max(g, 0) (1) or gelu in its tanh form (2). limit <= 0: no cap. Rows may be picked through `row_stride` (a row of the operand may be wider than 2 ff).
 __global__ void __launch_bounds__(DT_THREADS)
 capped_glu_kernel(void* __restrict__ out, int out_code, const void* __restrict__ gate_up, int in_code, int64_t row_stride,
-                  int ff, float limit, float slope, float up_shift, int64_t total, int relu) {
+                  int ff, float limit, float slope, float up_shift, int64_t total, int act) {
   const int64_t at = (int64_t)blockIdx.x * DT_THREADS + threadIdx.x;
   if (at >= total) return;
   const int64_t t = at / ff;
@@ -180,20 +187,51 @@ capped_glu_kernel(void* __restrict__ out, int out_code, const void* __restrict__
     g = fminf(g, limit);
     u = fminf(fmaxf(u, -limit), limit);
   }
-  // (`relu`: the gate passes where it is positive, max(g, 0) (u + up_shift), instead of through a sigmoid)
-  const float y = (relu ? fmaxf(g, 0.f) : g / (1.0f + expf(-slope * g))) * (u + up_shift);
-  dt_store(out, out_code, at, y);
+  dt_store(out, out_code, at, dt_gate(g, slope, act) * (u + up_shift));
+}
+
+// The same for sizes that are multiples of four: a thread takes four adjacent columns.
+template <typename TO>
+__global__ void __launch_bounds__(DT_THREADS)
+capped_glu_fours_kernel(TO* __restrict__ out, const float* __restrict__ gate_up, int64_t row_stride, int fours, float limit, float slope,
+                        float up_shift, int64_t total, int act) {
+  const int64_t at = (int64_t)blockIdx.x * DT_THREADS + threadIdx.x;
+  if (at >= total) return;
+  const int64_t t = at / fours;
+  const int i = 4 * (int)(at - t * fours);
+  const float4 gv = *(const float4*)(gate_up + t * row_stride + i), uv = *(const float4*)(gate_up + t * row_stride + 4 * fours + i);
+  const float g[4] = {gv.x, gv.y, gv.z, gv.w}, u[4] = {uv.x, uv.y, uv.z, uv.w};
+  float y[4];
+#pragma unroll
+  for (int k = 0; k < 4; ++k) {
+    const float gk = limit > 0.f ? fminf(g[k], limit) : g[k], uk = limit > 0.f ? fminf(fmaxf(u[k], -limit), limit) : u[k];
+    y[k] = dt_gate(gk, slope, act) * (uk + up_shift);
+  }
+  if constexpr (sizeof(TO) == 4) *(float4*)((float*)out + 4 * at) = make_float4(y[0], y[1], y[2], y[3]);
+  else
+    *(uint2*)((bf16_t*)out + 4 * at) = make_uint2((uint32_t)f2bf(y[0]) | ((uint32_t)f2bf(y[1]) << 16),
+                                                  (uint32_t)f2bf(y[2]) | ((uint32_t)f2bf(y[3]) << 16));
 }
 
 extern "C" int ts_capped_glu(void* out, int out_dtype, const void* gate_up, int in_dtype, int64_t row_stride, int n, int ff,
-                             float limit, float slope, float up_shift, int relu, hipStream_t stream) {
+                             float limit, float slope, float up_shift, int act, hipStream_t stream) {
   if (n <= 0) return TS_OK;
-  if (ff <= 0 || row_stride < 2 * (int64_t)ff) return TS_BAD_SHAPE;
+  if (ff <= 0 || row_stride < 2 * (int64_t)ff || act < 0 || act > 2) return TS_BAD_SHAPE;
   if ((out_dtype | in_dtype) & ~1) return TS_BAD_DTYPE;
   const int64_t total = (int64_t)n * ff;
   const int64_t blocks = (total + DT_THREADS - 1) / DT_THREADS;
   if (blocks > 0x7fffffff) return TS_BAD_SHAPE;
+  if (in_dtype == 0 && ff % 4 == 0 && row_stride % 4 == 0 && (((uintptr_t)out | (uintptr_t)gate_up) & 15) == 0) {
+    const unsigned groups = (unsigned)((total / 4 + DT_THREADS - 1) / DT_THREADS);
+    if (out_dtype == 0)
+      capped_glu_fours_kernel<float><<<groups, DT_THREADS, 0, stream>>>((float*)out, (const float*)gate_up, row_stride, ff / 4, limit, slope,
+                                                                        up_shift, total / 4, act);
+    else
+      capped_glu_fours_kernel<bf16_t><<<groups, DT_THREADS, 0, stream>>>((bf16_t*)out, (const float*)gate_up, row_stride, ff / 4, limit, slope,
+                                                                         up_shift, total / 4, act);
+    return ts_check_launch();
+  }
   capped_glu_kernel<<<(unsigned)blocks, DT_THREADS, 0, stream>>>(out, out_dtype, gate_up, in_dtype, row_stride, ff, limit, slope,
-                                                                 up_shift, total, relu);
+                                                                 up_shift, total, act);
   return ts_check_launch();
 }

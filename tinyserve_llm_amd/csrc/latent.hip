@@ -60,25 +60,62 @@ extern "C" int ts_segment_rmsnorm(void* out, int out_dtype, int64_t out_stride, 
 }
 
 // Two stretches of every row in one launch, in place (the norms over a token's whole q and whole k projection):
-// workgroup (row, 0) takes the first, (row, 1) the second.
+// workgroup (row, 0) takes the first, (row, 1) the second. With a bias (one number per column of the row) it is added
+// before the norms, and workgroup (row, 2) adds it to a third stretch, which has no norm. HELD > 0: a thread keeps its
+// elements of the stretch, up to that many, in registers between the two passes; 0: any size.
+template <int HELD>
 __global__ void __launch_bounds__(LT_THREADS)
 segment_rmsnorm_pair_kernel(float* __restrict__ x, int64_t x_stride, int off0, int size0, const float* __restrict__ w0, int off1,
-                            int size1, const float* __restrict__ w1, float eps) {
+                            int size1, const float* __restrict__ w1, float eps, const float* __restrict__ bias, int off2, int size2) {
   __shared__ float red[LT_WAVES];
-  const int off = blockIdx.y ? off1 : off0, size = blockIdx.y ? size1 : size0;
-  const float* weight = blockIdx.y ? w1 : w0;
+  const int which = blockIdx.y;
+  const int off = which == 0 ? off0 : which == 1 ? off1 : off2, size = which == 0 ? size0 : which == 1 ? size1 : size2;
+  const float* weight = which ? w1 : w0;
   float* row = x + (int64_t)blockIdx.x * x_stride + off;
+  const float* add = bias ? bias + off : nullptr;
+  if (which == 2) {
+    for (int d = threadIdx.x; d < size; d += LT_THREADS) row[d] += add[d];
+    return;
+  }
   float squares = 0.f;
-  for (int d = threadIdx.x; d < size; d += LT_THREADS) squares = fmaf(row[d], row[d], squares);
+  if constexpr (HELD > 0) {
+    float v[HELD], w[HELD];
+#pragma unroll
+    for (int j = 0; j < HELD; ++j) {
+      const int d = min((int)threadIdx.x + j * LT_THREADS, size - 1);
+      v[j] = row[d] + (add ? add[d] : 0.f);
+      w[j] = weight[d];
+    }
+#pragma unroll
+    for (int j = 0; j < HELD; ++j) squares = threadIdx.x + j * LT_THREADS < size ? fmaf(v[j], v[j], squares) : squares;
+    const float inv = 1.0f / sqrtf(lt_block_sum(squares, red) / (float)size + eps);
+#pragma unroll
+    for (int j = 0; j < HELD; ++j)
+      if (threadIdx.x + j * LT_THREADS < size) row[threadIdx.x + j * LT_THREADS] = v[j] * inv * w[j];
+    return;
+  }
+  for (int d = threadIdx.x; d < size; d += LT_THREADS) {
+    const float v = row[d] + (add ? add[d] : 0.f);
+    squares = fmaf(v, v, squares);
+  }
   const float inv = 1.0f / sqrtf(lt_block_sum(squares, red) / (float)size + eps);
-  for (int d = threadIdx.x; d < size; d += LT_THREADS) row[d] = row[d] * inv * weight[d];
+  for (int d = threadIdx.x; d < size; d += LT_THREADS) row[d] = (row[d] + (add ? add[d] : 0.f)) * inv * weight[d];
 }
 
 extern "C" int ts_segment_rmsnorm_pair(float* x, int64_t x_stride, int off0, int size0, const float* w0, int off1, int size1,
-                                       const float* w1, float eps, int num_rows, hipStream_t stream) {
+                                       const float* w1, float eps, const float* bias, int off2, int size2, int num_rows,
+                                       hipStream_t stream) {
   if (num_rows <= 0) return TS_OK;
   if (size0 <= 0 || size1 <= 0 || off0 < 0 || off1 < off0 + size0 || off1 + size1 > x_stride || !w0 || !w1) return TS_BAD_SHAPE;
-  segment_rmsnorm_pair_kernel<<<dim3(num_rows, 2), LT_THREADS, 0, stream>>>(x, x_stride, off0, size0, w0, off1, size1, w1, eps);
+  if (size2 > 0 && (!bias || off2 < off1 + size1 || off2 + size2 > x_stride)) return TS_BAD_SHAPE;
+  const dim3 grid(num_rows, size2 > 0 ? 3 : 2);
+#define LT_PAIR(HELD) segment_rmsnorm_pair_kernel<HELD><<<grid, LT_THREADS, 0, stream>>>(x, x_stride, off0, size0, w0, off1, size1, w1, eps, bias, off2, size2)
+  const int longest = size0 > size1 ? size0 : size1;
+  if (longest <= 4 * LT_THREADS) LT_PAIR(4);
+  else if (longest <= 8 * LT_THREADS) LT_PAIR(8);
+  else if (longest <= 16 * LT_THREADS) LT_PAIR(16);
+  else LT_PAIR(0);
+#undef LT_PAIR
   return ts_check_launch();
 }
 

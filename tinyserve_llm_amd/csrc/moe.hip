@@ -4,7 +4,9 @@
 //     divided by the chosen ones' sum (+ 1e-20) if `normalize`, times `scale`. With `softmax_chosen` the logits
 //     themselves are the scores, and the weights are the softmax over the chosen experts' logits alone. With
 //     `scoring` 2 the scores are the softmax over all the router's outputs. The router may have `extras` more rows
-//     than experts: their logits' sigmoids are left beside the choice (a gate on a shared expert, say).
+//     than experts: their logits' sigmoids are left beside the choice (a gate on a shared expert, say). With `groups` the
+//     experts form that many equal groups of neighbours, and only those of the `keep` groups whose best choice score is
+//     largest can be chosen.
 //   * `ts_moe_group`: the step's (token, choice) pairs grouped by expert, and the groups cut into tiles of rows
 //     that one workgroup of the product takes: [expert, first index, rows] per tile, rows 0 for the tiles of the
 //     launch that the step does not fill (the launch is sized for the worst case, so nothing comes back to the host).
@@ -31,7 +33,7 @@ template <typename TX>
 __global__ void __launch_bounds__(MOE_ROUTE_THREADS)
 moe_route_kernel(int32_t* __restrict__ ids_out, float* __restrict__ w_out, const TX* __restrict__ x,
                  const float* __restrict__ router, const float* __restrict__ correction, int num_tokens, int K, int E, int top,
-                 float scale, int normalize, int scoring, int extras, float* __restrict__ extra_out) {
+                 float scale, int normalize, int scoring, int extras, float* __restrict__ extra_out, int groups, int keep) {
   const bool softmax_chosen = scoring == 1;
   const int rows = E + extras;                            // rows of the router: the experts, then the extras
   extern __shared__ float lds[];
@@ -120,6 +122,22 @@ moe_route_kernel(int32_t* __restrict__ ids_out, float* __restrict__ w_out, const
     }
     wave_sync();
   }
+  if (groups > 1 && keep < groups) {
+    // lane g scores group g (groups <= 64); a group stays if fewer than `keep` beat it (ties: the lower group)
+    const int size = E / groups;
+    float best = -INFINITY;
+    if (lane < groups)
+      for (int e = lane * size; e < (lane + 1) * size; ++e) best = fmaxf(best, c_s[e]);
+    int ahead = 0;
+    for (int g = 0; g < groups; ++g) {
+      const float other = __shfl(best, g, TS_WAVE);
+      ahead += other > best || (other == best && g < lane);
+    }
+    wave_sync();
+    if (lane < groups && ahead >= keep)
+      for (int e = lane * size; e < (lane + 1) * size; ++e) c_s[e] = -INFINITY;
+    wave_sync();
+  }
   // lane j keeps the j-th choice (top <= 32 lanes of the 64)
   float my_pick = 0.f;
   int my_choice = 0;
@@ -156,19 +174,20 @@ moe_route_kernel(int32_t* __restrict__ ids_out, float* __restrict__ w_out, const
 
 extern "C" int ts_moe_route(int32_t* ids_out, float* w_out, const void* x, int x_dtype, const float* router,
                             const float* correction, int num_tokens, int K, int E, int top, float scale, int normalize,
-                            int scoring, int extras, float* extra_out, hipStream_t stream) {
+                            int scoring, int extras, float* extra_out, int groups, int keep, hipStream_t stream) {
   if (num_tokens <= 0) return TS_OK;
   if (K <= 0 || E <= 0 || E > MOE_MAX_EXPERTS || top <= 0 || top > MOE_MAX_TOP || top > E || scoring < 0 || scoring > 2 ||
-      extras < 0 || extras > TS_WAVE || (extras && !extra_out))
+      extras < 0 || extras > TS_WAVE || (extras && !extra_out) || groups < 1 || groups > TS_WAVE || E % groups || keep < 1 ||
+      keep > groups || top > keep * (E / groups))
     return TS_BAD_SHAPE;
   const unsigned blocks = (num_tokens + MOE_ROUTE_TOKENS - 1) / MOE_ROUTE_TOKENS;
   const size_t lds = (size_t)MOE_ROUTE_TOKENS * (2 * (E + extras) + MOE_ROUTE_CHUNK) * sizeof(float);
   if (x_dtype == 0)
     moe_route_kernel<float><<<blocks, MOE_ROUTE_THREADS, lds, stream>>>(ids_out, w_out, (const float*)x, router, correction,
-                                                                        num_tokens, K, E, top, scale, normalize, scoring, extras, extra_out);
+                                                                        num_tokens, K, E, top, scale, normalize, scoring, extras, extra_out, groups, keep);
   else if (x_dtype == 1)
     moe_route_kernel<bf16_t><<<blocks, MOE_ROUTE_THREADS, lds, stream>>>(ids_out, w_out, (const bf16_t*)x, router, correction,
-                                                                         num_tokens, K, E, top, scale, normalize, scoring, extras, extra_out);
+                                                                         num_tokens, K, E, top, scale, normalize, scoring, extras, extra_out, groups, keep);
   else return TS_BAD_DTYPE;
   return ts_check_launch();
 }

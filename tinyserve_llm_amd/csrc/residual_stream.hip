@@ -423,6 +423,28 @@ extern "C" int ts_scaled_sum(float* out, const float* a, float sa, const float* 
   return ts_check_launch();
 }
 
+// x = cap tanh(x / cap), in place
+__global__ void __launch_bounds__(RS_THREADS)
+soft_cap_kernel(float* __restrict__ x, float cap, int64_t total) {
+  const float inv = 1.0f / cap;
+  const int64_t fours = total / 4;
+  for (int64_t i = (int64_t)blockIdx.x * RS_THREADS + threadIdx.x; i < fours; i += (int64_t)gridDim.x * RS_THREADS) {
+    float4 v = ((const float4*)x)[i];
+    v.x = cap * tanhf(v.x * inv); v.y = cap * tanhf(v.y * inv); v.z = cap * tanhf(v.z * inv); v.w = cap * tanhf(v.w * inv);
+    ((float4*)x)[i] = v;
+  }
+  if (blockIdx.x == 0 && threadIdx.x < total % 4) x[4 * fours + threadIdx.x] = cap * tanhf(x[4 * fours + threadIdx.x] * inv);
+}
+
+extern "C" int ts_soft_cap(float* x, float cap, int64_t total, hipStream_t stream) {
+  if (total <= 0) return TS_OK;
+  if (!x || !(cap > 0.f) || ((uintptr_t)x & 15)) return TS_BAD_SHAPE;
+  int64_t blocks = (total / 4 + RS_THREADS) / RS_THREADS;
+  if (blocks > 16384) blocks = 16384;
+  soft_cap_kernel<<<(unsigned)blocks, RS_THREADS, 0, stream>>>(x, cap, total);
+  return ts_check_launch();
+}
+
 // out[t, j] = act(sums[t, j]) * table[ids[t], offset + j]: a gate's sums times a stretch of a token's row of a table
 __global__ void __launch_bounds__(RS_THREADS)
 gather_gate_kernel(void* __restrict__ out, int out_code, const float* __restrict__ sums, const void* __restrict__ table,

@@ -10,6 +10,8 @@
 //   * `ts_ssd_conv_keep`: leaves the convolution's last inputs in the slots (a step of single tokens does it in prepare).
 //   * `ts_ssd_step`: walks each request's tokens of the step in order with the state in registers; a request's state is
 //     read from its slot at the start and written back at the end. For decoded tokens, short portions, and 32-bit models.
+//     Step sizes and decays may also be one number per head for all tokens (`token_stride` 0), the decays then given
+//     themselves beside their logarithms (`keeps`), so that a long walk multiplies by exactly them.
 //   * `ts_ssd_chunks`: long portions in bfloat16, in chunks of 64 tokens on the matrix cores. With b_t the sum of l from
 //     the chunk's first token to t (every exponent below is <= 0) and S0 the state before the chunk,
 //         y_t = exp(b_t) S0 C_t + sum_{j <= t} exp(b_t - b_j) d_j (C_t . B_j) x_j + D x_t,
@@ -18,27 +20,11 @@
 //     element, and the read-outs. x, B and C are the operands as they are; what is 32-bit by nature (weighted x, the
 //     weights of the second sum, S0) enters a product as two bfloat16 terms.
 //   * `ts_gated_group_norm`: y silu(z), cut into equal parts, each divided by its own root mean square, times a weight.
-#include "attention_mfma.h"
+#include "chunk_ops.h"
 
 #define SS_THREADS 256
 #define SS_WAVES (SS_THREADS / TS_WAVE)
 #define SS_MAX_TAPS 16
-#define SS_L 64                 // tokens of a chunk
-#define SS_PAD 72               // a row of 64 tokens in shared memory: 16-byte pieces, rows four banks apart
-
-static __device__ __forceinline__ void ss_store4(float* p, const float (&v)[4]) { *(float4*)p = make_float4(v[0], v[1], v[2], v[3]); }
-static __device__ __forceinline__ void ss_store4(bf16_t* p, const float (&v)[4]) {
-  *(uint2*)p = make_uint2(pack_bf16(v[0], v[1]), pack_bf16(v[2], v[3]));
-}
-static __device__ __forceinline__ void ss_load4(const float* p, float (&v)[4]) {
-  const float4 x = *(const float4*)p;
-  v[0] = x.x; v[1] = x.y; v[2] = x.z; v[3] = x.w;
-}
-static __device__ __forceinline__ void ss_load4(const bf16_t* p, float (&v)[4]) {
-  const uint2 x = *(const uint2*)p;
-  v[0] = __uint_as_float(x.x << 16); v[1] = __uint_as_float(x.x & 0xffff0000u);
-  v[2] = __uint_as_float(x.y << 16); v[3] = __uint_as_float(x.y & 0xffff0000u);
-}
 
 struct SsSizes { int heads, vdim, vp, groups, state, np, taps; };
 
@@ -227,9 +213,9 @@ extern "C" int ts_ssd_conv_keep(float* kept, int64_t kept_stride, const float* p
 template <typename T, int NQ, int RV>
 __global__ void __launch_bounds__(SS_THREADS)
 ssd_step_kernel(float* __restrict__ out, const T* __restrict__ mixed, const float* __restrict__ steps, const float* __restrict__ logs,
-                const float* __restrict__ skip, float* __restrict__ states, int64_t slot_stride,
-                const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ state_slots, int heads, int vdim, int vp,
-                int groups, int up_to) {
+                const float* __restrict__ skip, const float* __restrict__ keeps, int token_stride, float* __restrict__ states,
+                int64_t slot_stride, const int32_t* __restrict__ cu_seqlens, const int32_t* __restrict__ state_slots, int heads,
+                int vdim, int vp, int groups, int up_to) {
   constexpr int np = 32 * NQ;
   const int seq = blockIdx.x, h = blockIdx.y;
   const int t_begin = cu_seqlens[seq], t_end = cu_seqlens[seq + 1];
@@ -238,7 +224,7 @@ ssd_step_kernel(float* __restrict__ out, const T* __restrict__ mixed, const floa
   const int row = heads * vp + 2 * groups * np, g = h / (heads / groups);
   const int b_at = heads * vp + g * np + 4 * part, c_at = b_at + groups * np;
   float* st = states + (int64_t)state_slots[seq] * slot_stride + (int64_t)h * vp * np + 4 * part;
-  const float d_skip = skip[h];
+  const float d_skip = skip ? skip[h] : 0.f, fixed_keep = keeps ? keeps[h] : 0.f;
   float S[RV][NQ][4];
 #pragma unroll
   for (int rv = 0; rv < RV; ++rv)
@@ -254,8 +240,8 @@ ssd_step_kernel(float* __restrict__ out, const T* __restrict__ mixed, const floa
     }
 #pragma unroll
     for (int rv = 0; rv < RV; ++rv) xn[rv] = Num<T>::ld(m + h * vp + min(v0 + 32 * rv, vp - 1));
-    dn = steps[(int64_t)t * heads + h];
-    ln = logs[(int64_t)t * heads + h];
+    dn = steps[(int64_t)t * token_stride + h];
+    ln = logs[(int64_t)t * token_stride + h];
   };
   fetch(t_begin);
   for (int t = t_begin; t < t_end; ++t) {
@@ -266,7 +252,7 @@ ssd_step_kernel(float* __restrict__ out, const T* __restrict__ mixed, const floa
       for (int k = 0; k < 4; ++k) B[i][k] = Bn[i][k], C[i][k] = Cn[i][k];
 #pragma unroll
     for (int rv = 0; rv < RV; ++rv) x[rv] = xn[rv];
-    const float d = dn, keep = expf(ln);
+    const float d = dn, keep = keeps ? fixed_keep : expf(ln);
     if (t + 1 < t_end) fetch(t + 1);
 #pragma unroll
     for (int rv = 0; rv < RV; ++rv) {
@@ -295,11 +281,12 @@ ssd_step_kernel(float* __restrict__ out, const T* __restrict__ mixed, const floa
 
 // states: each slot's S, float32 [heads, vp, np], `slot_stride` floats from slot to slot.
 extern "C" int ts_ssd_step(float* out, const void* mixed, int dtype, const float* steps, const float* logs, const float* skip,
-                           float* states, int64_t slot_stride, const int32_t* cu_seqlens, const int32_t* state_slots, int num_seqs,
+                           const float* keeps, int token_stride, float* states, int64_t slot_stride, const int32_t* cu_seqlens, const int32_t* state_slots, int num_seqs,
                            int heads, int vdim, int vp, int groups, int np, int up_to, hipStream_t stream) {
   if (num_seqs <= 0) return TS_OK;
   if (heads <= 0 || heads > 65535 || groups <= 0 || heads % groups || vdim <= 0 || vp < vdim || vp % 16 || np <= 0 || np % 32 || np > 512 ||
-      slot_stride < (int64_t)heads * vp * np || slot_stride % 4 || (((uintptr_t)states | (uintptr_t)mixed) & 15))
+      slot_stride < (int64_t)heads * vp * np || slot_stride % 4 || (((uintptr_t)states | (uintptr_t)mixed) & 15) ||
+      (token_stride != 0 && token_stride < heads))
     return TS_BAD_SHAPE;
   const int nq = np / 32;
   // (a slice of 64 rows where the step has workgroups enough and a lane's registers hold two rows' fours)
@@ -308,8 +295,8 @@ extern "C" int ts_ssd_step(float* out, const void* mixed, int dtype, const float
   if (slices > 65535) return TS_BAD_SHAPE;
   dim3 grid(num_seqs, heads, slices);
 #define SS_STEP(T, NQ, RV) \
-  ssd_step_kernel<T, NQ, RV><<<grid, SS_THREADS, 0, stream>>>(out, (const T*)mixed, steps, logs, skip, states, slot_stride, cu_seqlens, \
-                                                              state_slots, heads, vdim, vp, groups, up_to)
+  ssd_step_kernel<T, NQ, RV><<<grid, SS_THREADS, 0, stream>>>(out, (const T*)mixed, steps, logs, skip, keeps, token_stride, states, slot_stride, \
+                                                              cu_seqlens, state_slots, heads, vdim, vp, groups, up_to)
 #define SS_STEP_2(T, NQ) case NQ: if (rv == 2) SS_STEP(T, NQ, 2); else SS_STEP(T, NQ, 1); break;
 #define SS_STEP_1(T, NQ) case NQ: SS_STEP(T, NQ, 1); break;
 #define SS_STEP_N(T) \
@@ -329,58 +316,12 @@ extern "C" int ts_ssd_step(float* out, const void* mixed, int dtype, const float
 
 // ---- chunks of 64 tokens on the matrix cores (bfloat16) ----------------------------------------------------------
 
-// In the first wave, lane t: the running sum of the log decays up to token t of the chunk (tokens past its end add 0).
-// Differences of two such sums are what counts, and one token may decay by thousands where its neighbours hardly do: the
-// sums are 64-bit. A log decay below -128 counts as -128 (its exponential is 0 in 32-bit either way).
-static __device__ __forceinline__ double ss_running(const float* __restrict__ logs, int tok0, int len, int heads, int h) {
-  const int t = threadIdx.x;
-  double b = t < len ? (double)fmaxf(logs[(int64_t)(tok0 + t) * heads + h], -128.f) : 0.0;
-#pragma unroll
-  for (int off = 1; off < TS_WAVE; off <<= 1) {
-    const double up = __shfl_up(b, off, TS_WAVE);
-    if (t >= off) b += up;
-  }
-  return b;
-}
-
-static __device__ __forceinline__ uint4 ss_piece(const bf16_t* p, bool there) {
-  return there ? *(const uint4*)p : make_uint4(0, 0, 0, 0);
-}
-static __device__ __forceinline__ float ss_half(const uint4& p, int k) {
-  const uint32_t w = (&p.x)[k >> 1];
-  return __uint_as_float(k & 1 ? w & 0xffff0000u : w << 16);
-}
-static __device__ __forceinline__ uint32_t ss_rest(uint32_t hi, float a, float b) {
-  return pack_bf16(a - __uint_as_float(hi << 16), b - __uint_as_float(hi & 0xffff0000u));
-}
-
-// A tile of 64 tokens by 64 columns of `src` (rows `row` apart, columns at `col`, those from `cols` on absent) turned
-// round into dst[column][token]; as it is, or (WEIGHTED) times weight[token] in two terms.
-template <bool WEIGHTED>
-static __device__ __forceinline__ void ss_turn(bf16_t (*dst)[SS_PAD], bf16_t (*rest)[SS_PAD], const bf16_t* __restrict__ src, int row,
-                                               int tok0, int len, int cols, const float* weight) {
-  // a thread takes eight columns of two neighbouring tokens; neighbouring threads neighbouring pairs of tokens
-  const int pair = threadIdx.x & 31, p = threadIdx.x >> 5;
-  const int ta = 2 * pair, tb = ta + 1;
-  const bf16_t* at = src + (int64_t)tok0 * row + 8 * p;
-  const uint4 a = ss_piece(at + (int64_t)min(ta, len - 1) * row, ta < len && 8 * p < cols);
-  const uint4 b = ss_piece(at + (int64_t)min(tb, len - 1) * row, tb < len && 8 * p < cols);
-#pragma unroll
-  for (int k = 0; k < 8; ++k) {
-    float x = ss_half(a, k), y = ss_half(b, k);
-    if constexpr (WEIGHTED) x *= weight[ta], y *= weight[tb];
-    const uint32_t hi = pack_bf16(x, y);
-    *(uint32_t*)&dst[8 * p + k][ta] = hi;
-    if constexpr (WEIGHTED) *(uint32_t*)&rest[8 * p + k][ta] = ss_rest(hi, x, y);
-  }
-}
-
 // chunks: int32 [chunks, 4] (first token of the step, tokens 1 .. 64, request, whether the request's last). buf[chunk][head]
 // [vp][np] gets what the chunk adds to the state, totals[chunk][head] the chunk's whole log decay.
 __global__ void __launch_bounds__(SS_THREADS)
 ssd_chunk_sums_kernel(float* __restrict__ buf, float* __restrict__ totals, const bf16_t* __restrict__ mixed,
-                      const float* __restrict__ steps, const float* __restrict__ logs, const int32_t* __restrict__ chunks, int heads,
-                      int vp, int groups, int np) {
+                      const float* __restrict__ steps, const float* __restrict__ logs, int token_stride,
+                      const int32_t* __restrict__ chunks, int heads, int vp, int groups, int np) {
   __shared__ __attribute__((aligned(16))) bf16_t x_s[64][SS_PAD], xr_s[64][SS_PAD];     // weighted x, turned: [channel][token]
   __shared__ __attribute__((aligned(16))) bf16_t b_s[128][SS_PAD];                     // B, turned: [state][token]
   __shared__ float weight_s[SS_L];
@@ -389,9 +330,9 @@ ssd_chunk_sums_kernel(float* __restrict__ buf, float* __restrict__ totals, const
   const int row = heads * vp + 2 * groups * np, g = h / (heads / groups);
   const int wave = wave_index(), lane = threadIdx.x & (TS_WAVE - 1), r = lane & 15, q = lane >> 4;
   if (threadIdx.x < TS_WAVE) {
-    const double b = ss_running(logs, tok0, len, heads, h);
+    const double b = ss_running(logs, tok0, len, token_stride, h);
     const double total = __shfl(b, TS_WAVE - 1, TS_WAVE);
-    weight_s[lane] = lane < len ? expf((float)(total - b)) * steps[(int64_t)(tok0 + lane) * heads + h] : 0.f;
+    weight_s[lane] = lane < len ? expf((float)(total - b)) * steps[(int64_t)(tok0 + lane) * token_stride + h] : 0.f;
     if (lane == 0 && blockIdx.z == 0) totals[(int64_t)chunk * heads + h] = (float)total;
   }
   __syncthreads();
@@ -469,7 +410,7 @@ ssd_chunk_scan_kernel(float* __restrict__ buf, const float* __restrict__ totals,
 template <int NQ>
 __global__ void __launch_bounds__(SS_THREADS)
 ssd_chunk_out_kernel(float* __restrict__ out, const float* __restrict__ buf, const bf16_t* __restrict__ mixed,
-                     const float* __restrict__ steps, const float* __restrict__ logs, const float* __restrict__ skip,
+                     const float* __restrict__ steps, const float* __restrict__ logs, const float* __restrict__ skip, int token_stride,
                      const int32_t* __restrict__ chunks, int heads, int vdim, int vp, int groups) {
   constexpr int np = 32 * NQ;
   __shared__ __attribute__((aligned(16))) bf16_t x_s[64][SS_PAD];                      // x, turned: [channel][token]
@@ -484,8 +425,8 @@ ssd_chunk_out_kernel(float* __restrict__ out, const float* __restrict__ buf, con
   const bf16_t* b_rows = rows + heads * vp + g * np + 8 * q;
   const bf16_t* c_rows = b_rows + groups * np;
   if (threadIdx.x < TS_WAVE) {
-    b_s[lane] = ss_running(logs, tok0, len, heads, h);
-    d_s[lane] = lane < len ? steps[(int64_t)(tok0 + lane) * heads + h] : 0.f;
+    b_s[lane] = ss_running(logs, tok0, len, token_stride, h);
+    d_s[lane] = lane < len ? steps[(int64_t)(tok0 + lane) * token_stride + h] : 0.f;
   }
   ss_turn<false>(x_s, nullptr, mixed + h * vp + v0, row, tok0, len, vp - v0, nullptr);
   const int t = 16 * wave + r;                               // (this lane's token of the first product)
@@ -554,7 +495,7 @@ ssd_chunk_out_kernel(float* __restrict__ out, const float* __restrict__ buf, con
       acc[tb] = mfma32(lo, cf, acc[tb]);
     }
   }
-  const float d_skip = skip[h];
+  const float d_skip = skip ? skip[h] : 0.f;
   uint4 xf[2];
 #pragma unroll
   for (int k = 0; k < 2; ++k) xf[k] = *(const uint4*)&x_s[16 * wave + r][32 * k + 8 * q];
@@ -588,24 +529,25 @@ ssd_chunk_out_kernel(float* __restrict__ out, const float* __restrict__ buf, con
 }
 
 // buf float32 [chunks, heads, vp, np], totals float32 [chunks, heads].
-extern "C" int ts_ssd_chunks(float* out, const void* mixed, const float* steps, const float* logs, const float* skip, float* states,
-                             int64_t slot_stride, const int32_t* chunks, const int32_t* chunk_cu, const int32_t* state_slots,
+extern "C" int ts_ssd_chunks(float* out, const void* mixed, const float* steps, const float* logs, const float* skip, int token_stride,
+                             float* states, int64_t slot_stride, const int32_t* chunks, const int32_t* chunk_cu, const int32_t* state_slots,
                              float* buf, float* totals, int num_chunks, int num_seqs, int heads, int vdim, int vp, int groups, int np,
                              hipStream_t stream) {
   if (num_chunks <= 0 || num_seqs <= 0) return TS_OK;
   const int64_t per_head = (int64_t)vp * np;
   if (heads <= 0 || heads > 65535 || groups <= 0 || heads % groups || vdim <= 0 || vp < vdim || vp % 16 || np <= 0 || np % 32 || np > 512 ||
       per_head > (1 << 24) || slot_stride < heads * per_head || slot_stride % 4 ||
-      (((uintptr_t)states | (uintptr_t)mixed | (uintptr_t)buf | (uintptr_t)out) & 15))
+      (((uintptr_t)states | (uintptr_t)mixed | (uintptr_t)buf | (uintptr_t)out) & 15) || (token_stride != 0 && token_stride < heads))
     return TS_BAD_SHAPE;
   const int slices = (vp + 63) / 64;
   const int scan_blocks = (int)((per_head / 4 + SS_THREADS - 1) / SS_THREADS);
   const bf16_t* m = (const bf16_t*)mixed;
-  ssd_chunk_sums_kernel<<<dim3(num_chunks, heads, slices), SS_THREADS, 0, stream>>>(buf, totals, m, steps, logs, chunks, heads, vp, groups, np);
+  ssd_chunk_sums_kernel<<<dim3(num_chunks, heads, slices), SS_THREADS, 0, stream>>>(buf, totals, m, steps, logs, token_stride, chunks, heads, vp,
+                                                                                       groups, np);
   ssd_chunk_scan_kernel<<<dim3(num_seqs, heads, scan_blocks), SS_THREADS, 0, stream>>>(buf, totals, states, slot_stride, chunk_cu, state_slots,
                                                                                       heads, (int)per_head);
 #define SS_OUT(NQ) case NQ: ssd_chunk_out_kernel<NQ><<<dim3(num_chunks, heads, slices), SS_THREADS, 0, stream>>>( \
-    out, buf, m, steps, logs, skip, chunks, heads, vdim, vp, groups); break;
+    out, buf, m, steps, logs, skip, token_stride, chunks, heads, vdim, vp, groups); break;
   switch (np / 32) {
     SS_OUT(1) SS_OUT(2) SS_OUT(3) SS_OUT(4) SS_OUT(5) SS_OUT(6) SS_OUT(7) SS_OUT(8) SS_OUT(9) SS_OUT(10) SS_OUT(11) SS_OUT(12)
     SS_OUT(13) SS_OUT(14) SS_OUT(15) SS_OUT(16)

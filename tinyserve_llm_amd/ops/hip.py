@@ -83,7 +83,7 @@ def _declare(lib: ctypes.CDLL) -> None:
         "ts_bias_activation": [p, i, p, i, p, i, i, i, i, p],
         "ts_mingru_scan": [p, i, p, i, p, i, p, p, p, i, i, i, p],
         "ts_mingru_scan_chunks": [p, i, p, i, p, i, p, p, p, p, p, i, i, i, p],
-        "ts_qkv_finish": [p, p, p, p, p, p, p, i, i, i, i, i, i, i, i, f, i, f, i, i64, i64, i64, i64, i64, i64, i64, i, i, f, p],
+        "ts_qkv_finish": [p, p, p, p, p, p, p, i, i, i, i, i, i, i, i, f, i, f, i, i64, i64, i64, i64, i64, i64, i64, i, i, f, i64, p],
         "ts_paged_attention_general": [p, p, p, p, p, p, p, i, i, i, i, i, i, i64, i64, i64, i64, i64, i64, i64, i, f, f, i, i,
                                        i, i, p, p, p, i64, p],
         "ts_dyt": [p, i, p, i, p, i, p, i, p, p, p, p, i, i, p],
@@ -93,11 +93,11 @@ def _declare(lib: ctypes.CDLL) -> None:
         "ts_conv_finish": [p, p, p, p, i64, p, p, p, p, f, p, p, p, p, p, i, i, i, i, i, i, f, i, i, i64, i64, i64, i64, i64,
                            i64, i64, i, i, i, p],
         "ts_conv_state_update": [p, p, i64, p, p, i, i, i, i, p],
-        "ts_moe_route": [p, p, p, i, p, p, i, i, i, i, f, i, i, i, p, p],
+        "ts_moe_route": [p, p, p, i, p, p, i, i, i, i, f, i, i, i, p, i, i, p],
         "ts_moe_group": [p, p, p, i, i, i, i, p],
         "ts_moe_gemm": [p, i, p, i, p, p, p, i, i, i, i, i, i, f, f, f, i, p],
         "ts_segment_rmsnorm": [p, i, i64, p, i64, i, p, f, i, p],
-        "ts_segment_rmsnorm_pair": [p, i64, i, i, p, i, i, p, f, i, p],
+        "ts_segment_rmsnorm_pair": [p, i64, i, i, p, i, i, p, f, p, i, i, i, p],
         "ts_latent_finish": [p, p, i, p, i64, i, i, i, i, i, p, p, f, p, f, p, p, i, i64, i64, p, i64, i64, i, p],
         "ts_latent_mfma_takes": [i, i],
         "ts_heads_gemm_mfma": [p, i, i64, i64, p, i, i64, i64, p, i64, i64, i, i, i, i, p, i64, p],
@@ -109,8 +109,13 @@ def _declare(lib: ctypes.CDLL) -> None:
         "ts_stream_join": [p, i, p, p, i, p, i, p, i, i, p],
         "ts_ssd_prepare": [p, i, p, p, p, i64, p, p, p, i64, p, p, p, p, p, i, i, i, i, i, i, i, i, i, p],
         "ts_ssd_conv_keep": [p, i64, p, i64, p, p, i, i, i, i, i, i, i, i, p],
-        "ts_ssd_step": [p, p, i, p, p, p, p, i64, p, p, i, i, i, i, i, i, i, p],
-        "ts_ssd_chunks": [p, p, p, p, p, p, i64, p, p, p, p, p, i, i, i, i, i, i, i, p],
+        "ts_ssd_step": [p, p, i, p, p, p, p, i, p, i64, p, p, i, i, i, i, i, i, i, p],
+        "ts_ssd_chunks": [p, p, p, p, p, i, p, i64, p, p, p, p, p, i, i, i, i, i, i, i, p],
+        "ts_retention_prepare": [p, i, p, i64, p, p, i, i, i, i, i, i, i, p],
+        "ts_delta_prepare": [p, i, p, p, p, p, i64, p, p, i64, p, p, p, p, p, i, i, i, i, i, i, i, i, f, i, p],
+        "ts_delta_step": [p, p, i, p, p, p, p, i64, p, p, i, i, i, i, i, i, i, p],
+        "ts_delta_chunks": [p, p, p, p, p, p, i64, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, p],
+        "ts_soft_cap": [p, f, i64, p],
         "ts_gated_group_norm": [p, i, p, p, i64, p, i, i, i, f, p],
         "ts_mlstm_scan": [p, p, i64, p, p, p, p, p, i, i, i, i, i, f, f, p],
         "ts_mlstm_scan_chunks": [p, p, i64, p, p, p, p, p, p, p, p, p, i, i, i, i, i, f, f, p],
@@ -439,7 +444,7 @@ def paged_attention_decode(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torc
         part_o = torch.empty((T, nh, splits, hd), dtype=torch.float32, device=q.device)
         part_ml = torch.empty((T, nh, splits, 2), dtype=torch.float32, device=q.device)
     general = softcap > 0 or sink or sinks is not None or slopes is not None or gate is not None
-    gate_stride = _check_gate(gate, q.shape[0], q.shape[1] * q.shape[2])
+    gate_stride = _check_heads_gate(gate, q.shape[0], q.shape[1], q.shape[2])
     leave_split = leave_split and not general and out is None and 1 < splits <= SPLIT_ATTENTION_MAX_CHUNKS
     out = None if leave_split else _out_like(q, out)
     if general:
@@ -734,7 +739,7 @@ def paged_attention_prefill(q: torch.Tensor, k_cache: torch.Tensor, v_cache: tor
         _gpu(gate)
         _run("paged_attention_prefill_general", library().ts_paged_attention_prefill_general(
             *args, float(softcap), int(sink), _ptr(sinks), _ptr(slopes), _ptr(gate),
-            _check_gate(gate, q.shape[0], q.shape[1] * q.shape[2]), _stream()))
+            _check_heads_gate(gate, q.shape[0], q.shape[1], q.shape[2]), _stream()))
     else:
         _run("paged_attention_prefill", library().ts_paged_attention_prefill(*args, _stream()))
     return out
@@ -753,7 +758,8 @@ def paged_attention(q: torch.Tensor, k_cache: torch.Tensor, v_cache: torch.Tenso
     back to `paged_attention_general`, which is 32-bit throughout. `sinks` / `slopes` (float32 [heads]): learned
     sinks (exp(sinks[h]) in the denominator) and a penalty of slopes[h] per position of distance on every score,
     by the general variants likewise. `gate` (float32 [tokens, heads * value_dim], rows may lie apart): the
-    output is multiplied element by element by sigmoid(gate) on its way out of whichever kernel writes it.
+    output is multiplied element by element by sigmoid(gate) on its way out of whichever kernel writes it; float32
+    [tokens, heads]: each head's output by its one number.
     `chunk_mask` > 0 (instead of `window`): a position sees the keys of its own chunk of that many positions,
     chunks counted from position 0 of the request; the kernels take it as a window below zero."""
     _need(chunk_mask >= 0 and window >= 0 and not (chunk_mask and window), "a sliding window or chunks, both counted in positions")
@@ -1770,7 +1776,7 @@ def qkv_finish(qkv: torch.Tensor, freqs: torch.Tensor | None, positions: torch.T
                k_cache: torch.Tensor | None, v_cache: torch.Tensor | None, num_heads: int, num_kv_heads: int,
                head_dim: int, value_dim: int, out_dtype: torch.dtype, *, interleaved: bool = True,
                qk_norm_eps: float | None = None, v_norm_eps: float | None = None, amplitude: float = 1.0) -> torch.Tensor:
-    """From a projected row q | k | v ([tokens, nh hd + nkv hd + nkv vd], float32 or `out_dtype`) to q
+    """From a projected row q | k | v ([tokens, >= nh hd + nkv hd + nkv vd], float32 or `out_dtype`) to q
     [tokens, nh, hd] and the cache slots of k and v, in `out_dtype`. `freqs` (float64 [rot / 2]): q and
     k turn in their first rot dimensions by position * freqs[i], pair i being dimensions (2i, 2i+1) if
     `interleaved`, else (i, i + rot/2), cosine and sine times `amplitude`. `qk_norm_eps` / `v_norm_eps`: each q
@@ -1778,7 +1784,7 @@ def qkv_finish(qkv: torch.Tensor, freqs: torch.Tensor | None, positions: torch.T
     _gpu(qkv, freqs, positions, slots, k_cache, v_cache)
     T = qkv.shape[0]
     row = (num_heads + num_kv_heads) * head_dim + num_kv_heads * value_dim
-    _need(qkv.dim() == 2 and qkv.shape[1] == row and qkv.is_contiguous(), lambda: f"qkv must be contiguous [tokens, {row}]")
+    _need(qkv.dim() == 2 and qkv.shape[1] >= row and qkv.is_contiguous(), lambda: f"qkv must be contiguous [tokens, >= {row}]")
     _need(qkv.dtype in (torch.float32, out_dtype), "the projected rows are float32 or of the output's type")
     _need(0 < head_dim <= 256 and 0 < value_dim <= 256, "head sizes up to 256")
     _need(positions.dtype == torch.int32 and positions.shape == (T,) and positions.is_contiguous(), "positions must be int32 [tokens]")
@@ -1798,7 +1804,7 @@ def qkv_finish(qkv: torch.Tensor, freqs: torch.Tensor | None, positions: torch.T
         _ptr(q), _ptr(k_cache), _ptr(v_cache), _ptr(qkv), _ptr(freqs), _ptr(positions), _ptr(slots), T, num_heads,
         num_kv_heads, head_dim, value_dim, rot, int(interleaved), int(qk_norm_eps is not None), float(qk_norm_eps or 0.0),
         int(v_norm_eps is not None), float(v_norm_eps or 0.0), page_size, *kst, *vst, _code(qkv.dtype), _code(out_dtype),
-        float(amplitude), _stream()))
+        float(amplitude), qkv.shape[1], _stream()))
     return q
 
 
@@ -1812,10 +1818,10 @@ def paged_attention_general(q: torch.Tensor, k_cache: torch.Tensor, v_cache: tor
     Value rows may differ in size from key rows: out [tokens, heads, value_dim]. `sinks` (float32 [heads]):
     the sink's score is sinks[h] instead of 0; `slopes` (float32 [heads]): slopes[h] * (query position - key
     position) is taken off every score; `gate` (float32 [tokens, heads * value_dim], a view whose rows may lie
-    apart): the output row is multiplied by sigmoid(gate) element by element."""
+    apart): the output row is multiplied by sigmoid(gate) element by element; or [tokens, heads], one number per head."""
     _gpu(q, k_cache, v_cache, block_tables, seq_of_token, positions, sinks, slopes, gate)
     _check_head_vectors(q.shape[1], sinks, slopes)
-    gate_stride = _check_gate(gate, q.shape[0], q.shape[1] * v_cache.shape[3])
+    gate_stride = _check_heads_gate(gate, q.shape[0], q.shape[1], v_cache.shape[3])
     _need(q.dim() == 3 and q.is_contiguous(), "q must be contiguous [tokens, heads, head_dim]")
     T, nh, hd = q.shape
     nkv, vd = k_cache.shape[2], v_cache.shape[3]
@@ -1846,6 +1852,14 @@ def _check_gate(gate: torch.Tensor | None, tokens: int, width: int) -> int:
     _need(gate.dtype == torch.float32 and gate.dim() == 2 and gate.shape == (tokens, width) and gate.stride(1) == 1
           and gate.stride(0) >= width, "the gate must be float32 [tokens, heads * value_dim] with contiguous rows")
     return gate.stride(0)
+
+
+def _check_heads_gate(gate: torch.Tensor | None, tokens: int, heads: int, vdim: int) -> int:
+    """The stride between the rows of a gate on attention's output: a number per element ([tokens, heads vdim]), or one per
+    head ([tokens, heads]), which the kernels know by a stride below zero."""
+    if gate is None or gate.dim() != 2 or gate.shape[1] != heads or vdim == 1:
+        return _check_gate(gate, tokens, heads * vdim)
+    return -_check_gate(gate, tokens, heads)
 
 
 # ---- the dynamic-tanh norm ----
@@ -1916,18 +1930,22 @@ def embedding_dyt_stream(table: torch.Tensor, ids: torch.Tensor, scale: float = 
     return out
 
 
+GLU_ACTIVATIONS = {"sigmoid": 0, "relu": 1, "gelu_tanh": 2}
+
+
 def capped_glu(gate_up: torch.Tensor, limit: float, slope: float, up_shift: float, out_dtype: torch.dtype,
-               relu: bool = False) -> torch.Tensor:
+               activation: str = "sigmoid") -> torch.Tensor:
     """From rows [gate | up] (float32 or `out_dtype`): g = min(gate, limit), u = clamp(up, -limit, limit)
-    (limit <= 0: no cap), y = g sigmoid(slope g) (u + up_shift), or max(g, 0) (u + up_shift) with `relu`, in 32-bit,
-    stored as `out_dtype`."""
+    (limit <= 0: no cap), y = act(g) (u + up_shift) in 32-bit, stored as `out_dtype`; act(g) is g sigmoid(slope g)
+    ("sigmoid"), max(g, 0) ("relu") or gelu in its tanh form ("gelu_tanh")."""
     _gpu(gate_up)
+    _need(activation in GLU_ACTIVATIONS, lambda: f"activation {activation!r}: one of {sorted(GLU_ACTIVATIONS)}")
     _need(gate_up.dim() == 2 and gate_up.shape[1] % 2 == 0 and gate_up.stride(1) == 1 and gate_up.stride(0) >= gate_up.shape[1],
           "the input must be [tokens, 2 ff] with contiguous rows")
     n, ff = gate_up.shape[0], gate_up.shape[1] // 2
     out = torch.empty((n, ff), dtype=out_dtype, device=gate_up.device)
     _run("capped_glu", library().ts_capped_glu(_ptr(out), _code(out_dtype), _ptr(gate_up), _code(gate_up.dtype), gate_up.stride(0),
-                                               n, ff, float(limit), float(slope), float(up_shift), int(relu), _stream()))
+                                               n, ff, float(limit), float(slope), float(up_shift), GLU_ACTIVATIONS[activation], _stream()))
     return out
 
 
@@ -2017,16 +2035,20 @@ MOE_WIDE_TILE_ROWS = 64   # or, in bfloat16, where the experts have this many ro
 MOE_LDS_TILE_ROWS = 128   # or this many (both operands then go through LDS; reductions that are multiples of 64)
 MOE_MAX_EXPERTS = 1024
 MOE_MAX_TOP = 32
+MOE_MAX_GROUPS = 64
 
 
 def moe_route(x: torch.Tensor, router: torch.Tensor, correction: torch.Tensor | None, top: int, scale: float,
-              normalize: bool = True, softmax_chosen: bool = False, softmax_all: bool = False, extras: int = 0):
+              normalize: bool = True, softmax_chosen: bool = False, softmax_all: bool = False, extras: int = 0,
+              groups: tuple[int, int] = (1, 1)):
     """(experts int32 [tokens, top], weights float32 [tokens, top]): scores s = sigmoid(x · routerᵀ) in 32-bit;
     the `top` experts with the largest s + correction; weights s of the chosen, over their sum (+ 1e-20) if
     `normalize`, times `scale`. `softmax_chosen`: the logits themselves are the scores, and the weights are the
     softmax over the chosen experts' logits alone (times `scale`). `softmax_all`: the scores are the softmax over
     all the experts' logits. `extras`: the router's last rows beyond the experts, whose logits' sigmoids come back as
-    a third result, float32 [tokens, extras] (a gate on a shared expert, say)."""
+    a third result, float32 [tokens, extras] (a gate on a shared expert, say). `groups` = (count, keep): the experts form
+    `count` equal groups of neighbours, and only those of the `keep` groups whose best choice score (s + correction) is
+    largest can be chosen."""
     _gpu(x, router, correction)
     _need(x.dim() == 2 and x.is_contiguous(), "the input must be contiguous [tokens, width]")
     _need(0 <= extras < router.shape[0] and extras <= 64 and not (softmax_chosen and softmax_all), "up to 64 extra rows; one way of scoring")
@@ -2035,12 +2057,15 @@ def moe_route(x: torch.Tensor, router: torch.Tensor, correction: torch.Tensor | 
     _need(correction is None or (correction.dtype == torch.float32 and correction.shape == (E,) and correction.is_contiguous()),
           "the correction must be float32 [experts]")
     _need(1 <= top <= min(E, MOE_MAX_TOP) and E <= MOE_MAX_EXPERTS, lambda: f"1 <= top <= min(experts, {MOE_MAX_TOP}), experts <= {MOE_MAX_EXPERTS}")
+    count, keep = groups
+    _need(1 <= keep <= count <= MOE_MAX_GROUPS and E % count == 0 and top <= keep * (E // count),
+          lambda: f"{E} experts in up to {MOE_MAX_GROUPS} equal groups, of which those kept hold at least {top}")
     ids = torch.empty((x.shape[0], top), dtype=torch.int32, device=x.device)
     weights = torch.empty((x.shape[0], top), dtype=torch.float32, device=x.device)
     extra = torch.empty((x.shape[0], extras), dtype=torch.float32, device=x.device) if extras else None
     _run("moe_route", library().ts_moe_route(_ptr(ids), _ptr(weights), _ptr(x), _code(x.dtype), _ptr(router), _ptr(correction),
                                              x.shape[0], x.shape[1], E, top, float(scale), int(normalize),
-                                             2 if softmax_all else int(softmax_chosen), extras, _ptr(extra), _stream()))
+                                             2 if softmax_all else int(softmax_chosen), extras, _ptr(extra), count, keep, _stream()))
     return (ids, weights, extra) if extras else (ids, weights)
 
 
@@ -2151,17 +2176,24 @@ def segment_rmsnorm(x: torch.Tensor, offset: int, size: int, weight: torch.Tenso
     return out
 
 
-def segment_rmsnorm_pair(x: torch.Tensor, first: tuple[int, int, torch.Tensor], second: tuple[int, int, torch.Tensor], eps: float) -> None:
+def segment_rmsnorm_pair(x: torch.Tensor, first: tuple[int, int, torch.Tensor], second: tuple[int, int, torch.Tensor], eps: float,
+                         bias: torch.Tensor | None = None, rest: tuple[int, int] = (0, 0)) -> None:
     """Two stretches (offset, size, weight float32 [size]) of every row of x (contiguous float32 [rows, width]), the second
-    behind the first, each divided by its own root mean square and multiplied by its weight, in place, in one launch."""
-    _gpu(x, first[2], second[2])
+    behind the first, each divided by its own root mean square and multiplied by its weight, in place, in one launch. `bias`
+    (float32, a number per column up to the last stretch's end) is added before the norms, and to the stretch `rest`
+    (offset, size) behind them, which has no norm."""
+    _gpu(x, first[2], second[2], bias)
     _need(x.dtype == torch.float32 and x.dim() == 2 and x.is_contiguous(), "contiguous rows of float32")
     for off, size, w in (first, second):
         _need(w.dtype == torch.float32 and w.shape == (size,) and w.is_contiguous(), "a weight must be float32 [size]")
     _need(0 <= first[0] and first[1] > 0 and second[1] > 0 and first[0] + first[1] <= second[0] and second[0] + second[1] <= x.shape[1],
           "two stretches inside a row, one behind the other")
+    end = max(second[0] + second[1], rest[0] + rest[1])
+    _need(rest[1] == 0 or (bias is not None and rest[1] > 0 and second[0] + second[1] <= rest[0] and end <= x.shape[1]),
+          "a further stretch lies behind the two, inside the row, and is there for its bias")
+    _need(bias is None or (bias.dtype == torch.float32 and bias.dim() == 1 and bias.shape[0] >= end and bias.is_contiguous()), "the bias must be float32, a number per column")
     _run("segment_rmsnorm_pair", library().ts_segment_rmsnorm_pair(_ptr(x), x.shape[1], first[0], first[1], _ptr(first[2]), second[0], second[1],
-                                                                   _ptr(second[2]), float(eps), x.shape[0], _stream()))
+                                                                   _ptr(second[2]), float(eps), _ptr(bias), rest[0], rest[1], x.shape[0], _stream()))
 
 
 def _check_step_vectors(T: int, **vectors: torch.Tensor | None) -> None:
@@ -2426,19 +2458,19 @@ def mlstm_scan(proj: torch.Tensor, i_bias: torch.Tensor, f_bias: torch.Tensor, s
     return out
 
 
-def mlstm_finish(o: torch.Tensor, weight: torch.Tensor, gate: torch.Tensor, heads: int, vdim: int, eps: float, out_dtype: torch.dtype,
+def mlstm_finish(o: torch.Tensor, weight: torch.Tensor | None, gate: torch.Tensor, heads: int, vdim: int, eps: float, out_dtype: torch.dtype,
                  silu_gate: bool = False) -> torch.Tensor:
     """Each head's row of o (float32 [tokens, heads vdim]) divided by its root mean square, times `weight` (float32
-    [heads vdim], or [vdim]: one weight that all heads share), times sigmoid(gate) (float32 [tokens, heads vdim], rows
+    [heads vdim], or [vdim]: one weight that all heads share; None: none), times sigmoid(gate) (float32 [tokens, heads vdim], rows
     may lie apart; with `silu_gate` times gate sigmoid(gate)), as `out_dtype`."""
     _gpu(o, weight, gate)
     T = o.shape[0]
     _need(o.dtype == torch.float32 and o.shape == (T, heads * vdim) and o.is_contiguous(), "o must be contiguous float32 [tokens, heads vdim]")
-    _need(weight.dtype == torch.float32 and weight.shape in ((heads * vdim,), (vdim,)) and weight.is_contiguous(),
+    _need(weight is None or (weight.dtype == torch.float32 and weight.shape in ((heads * vdim,), (vdim,)) and weight.is_contiguous()),
           "the weight must be float32 [heads vdim], or [vdim] for all heads")
     out = torch.empty((T, heads * vdim), dtype=out_dtype, device=o.device)
     _run("mlstm_finish", library().ts_mlstm_finish(_ptr(out), _code(out_dtype), _ptr(o), _ptr(weight), _ptr(gate), _check_gate(gate, T, heads * vdim),
-                                                   T, heads, vdim, float(eps), vdim if weight.shape[0] == heads * vdim else 0, int(silu_gate),
+                                                   T, heads, vdim, float(eps), vdim if weight is not None and weight.shape[0] == heads * vdim else 0, int(silu_gate),
                                                    _stream()))
     return out
 
@@ -2672,17 +2704,41 @@ def ssd_chunk_lists(host_cu_seqlens: list[int], from_tokens: int) -> tuple[list[
     return flat, cu
 
 
-def ssd_scan(mixed: torch.Tensor, steps: torch.Tensor, logs: torch.Tensor, skip: torch.Tensor, state: torch.Tensor, ctx,
-             sizes: SsdSizes, chunks_from: int = SSD_CHUNKS_FROM) -> torch.Tensor:
+def _step_chunks(ctx, from_tokens: int, device) -> "tuple[torch.Tensor, torch.Tensor]":
+    """`ssd_chunk_lists` of a step on the device (int32 [chunks, 4] and [requests + 1]), made once and kept in the step's scratch."""
+    kept = ctx.scratch.get(("ssd_chunks", from_tokens))
+    if kept is None:
+        # (a list copied from the host while a graph is being recorded would be read again, from memory long freed, at every replay)
+        _need(not torch.cuda.is_current_stream_capturing(), "the chunk list is made before a graph is recorded")
+        _need(len(ctx.host_cu_seqlens) == ctx.num_seqs + 1 and ctx.host_cu_seqlens[-1] == ctx.num_tokens, "the host's lengths are the step's")
+        flat, cu = ssd_chunk_lists(ctx.host_cu_seqlens, from_tokens)
+        kept = (torch.tensor(flat, dtype=torch.int32).view(-1, 4).to(device, non_blocking=True),
+                torch.tensor(cu, dtype=torch.int32).to(device, non_blocking=True))
+        ctx.scratch[("ssd_chunks", from_tokens)] = kept
+    return kept
+
+
+def _all_in_chunks(ctx, from_tokens: int) -> bool:
+    return all(b - a >= from_tokens for a, b in zip(ctx.host_cu_seqlens, ctx.host_cu_seqlens[1:]))
+
+
+def ssd_scan(mixed: torch.Tensor, steps: torch.Tensor, logs: torch.Tensor, skip: torch.Tensor | None, state: torch.Tensor, ctx,
+             sizes: SsdSizes, chunks_from: int = SSD_CHUNKS_FROM, keeps: torch.Tensor | None = None) -> torch.Tensor:
     """The recurrence over a packed step: per head S <- exp(log) S + step x B^T, y = S C + skip x, each request from and to
     its slot of `state` (S [heads, vp, np] at the start of the slot's row). mixed, steps, logs as `ssd_prepare` leaves
-    them, skip float32 [heads]. Returns y float32 [tokens, heads vdim]. In bfloat16, requests that feed at least
-    `chunks_from` tokens are worked in chunks on the matrix cores; all others, and 32-bit rows always, token by token."""
-    _gpu(mixed, steps, logs, skip, state)
+    them, skip float32 [heads] (None: no such term). Returns y float32 [tokens, heads vdim]. In bfloat16, requests that feed at
+    least `chunks_from` tokens are worked in chunks on the matrix cores; all others, and 32-bit rows always, token by token.
+    `keeps` (float32 [heads]): every token of a head has the same decay, this one; steps and logs (its logarithm) are then
+    [heads] as well."""
+    _gpu(mixed, steps, logs, skip, state, keeps)
     z, T = sizes, mixed.shape[0]
     _need(mixed.shape == (T, z.row) and mixed.is_contiguous(), lambda: f"the mixed rows must be contiguous [tokens, {z.row}]")
-    for t in (steps, logs):
-        _need(t.dtype == torch.float32 and t.shape == (T, z.heads) and t.is_contiguous(), "steps and logs must be float32 [tokens, heads]")
+    if keeps is not None:
+        _check_head_vectors(z.heads, steps, logs, keeps)
+    else:
+        for t in (steps, logs):
+            _need(t.dtype == torch.float32 and t.shape == (T, z.heads) and t.is_contiguous(), "steps and logs must be float32 [tokens, heads]")
+    token_stride = z.heads if keeps is None else 0
     _check_head_vectors(z.heads, skip)
     _check_ssd_state(state, z)
     _check_step_requests(ctx)
@@ -2691,27 +2747,18 @@ def ssd_scan(mixed: torch.Tensor, steps: torch.Tensor, logs: torch.Tensor, skip:
     out = torch.empty((T, z.inner), dtype=torch.float32, device=mixed.device)
     chunked = mixed.dtype == torch.bfloat16 and ctx.max_query_len >= chunks_from
     if chunked:
-        kept = ctx.scratch.get(("ssd_chunks", chunks_from))
-        if kept is None:
-            # (a list copied from the host while a graph is being recorded would be read again, from memory long freed, at every replay)
-            _need(not torch.cuda.is_current_stream_capturing(), "the chunk list is made before a graph is recorded")
-            _need(len(ctx.host_cu_seqlens) == S + 1 and ctx.host_cu_seqlens[-1] == T, "the host's lengths are the step's")
-            flat, cu = ssd_chunk_lists(ctx.host_cu_seqlens, chunks_from)
-            kept = (torch.tensor(flat, dtype=torch.int32).view(-1, 4).to(mixed.device, non_blocking=True),
-                    torch.tensor(cu, dtype=torch.int32).to(mixed.device, non_blocking=True))
-            ctx.scratch[("ssd_chunks", chunks_from)] = kept
-        chunks, chunk_cu = kept
+        chunks, chunk_cu = _step_chunks(ctx, chunks_from, mixed.device)
         C = chunks.shape[0]
         buf = torch.empty((C, z.matrix), dtype=torch.float32, device=mixed.device)
         totals = torch.empty((C, z.heads), dtype=torch.float32, device=mixed.device)
         _run("ssd_chunks", library().ts_ssd_chunks(
-            _ptr(out), _ptr(mixed), _ptr(steps), _ptr(logs), _ptr(skip), _ptr(state), state.stride(0), _ptr(chunks), _ptr(chunk_cu),
+            _ptr(out), _ptr(mixed), _ptr(steps), _ptr(logs), _ptr(skip), token_stride, _ptr(state), state.stride(0), _ptr(chunks), _ptr(chunk_cu),
             _ptr(ctx.state_slots), _ptr(buf), _ptr(totals), C, S, z.heads, z.vdim, z.vp, z.groups, z.np, _stream()))
-        if all(b - a >= chunks_from for a, b in zip(ctx.host_cu_seqlens, ctx.host_cu_seqlens[1:])):
+        if _all_in_chunks(ctx, chunks_from):
             return out
     _run("ssd_step", library().ts_ssd_step(
-        _ptr(out), _ptr(mixed), _code(mixed.dtype), _ptr(steps), _ptr(logs), _ptr(skip), _ptr(state), state.stride(0), _ptr(ctx.cu_seqlens),
-        _ptr(ctx.state_slots), S, z.heads, z.vdim, z.vp, z.groups, z.np, chunks_from - 1 if chunked else 0, _stream()))
+        _ptr(out), _ptr(mixed), _code(mixed.dtype), _ptr(steps), _ptr(logs), _ptr(skip), _ptr(keeps), token_stride, _ptr(state), state.stride(0),
+        _ptr(ctx.cu_seqlens), _ptr(ctx.state_slots), S, z.heads, z.vdim, z.vp, z.groups, z.np, chunks_from - 1 if chunked else 0, _stream()))
     return out
 
 
@@ -2726,3 +2773,116 @@ def gated_group_norm(y: torch.Tensor, gate: torch.Tensor, weight: torch.Tensor, 
     _run("gated_group_norm", library().ts_gated_group_norm(_ptr(out), _code(out_dtype), _ptr(y), _ptr(gate), _check_gate(gate, T, width), _ptr(weight),
                                                            T, width, parts, float(eps), _stream()))
     return out
+
+
+# ---- retention and the gated delta rule, on the places of a state-space mixer ----
+
+def retention_prepare(proj: torch.Tensor, freqs: torch.Tensor | None, positions: torch.Tensor, sizes: SsdSizes, out_dtype: torch.dtype) -> torch.Tensor:
+    """From projected rows (float32 [tokens, >= heads (vdim + 2 dim)], v | k | q leading) to the mixed rows that `ssd_scan`
+    reads (x = v, B = k, C = q, a group per head), as `out_dtype`: k and q turned by the token's position in their first
+    2 len(freqs) dimensions, pairs (i, i + len(freqs)), `freqs` float64 (None: nothing turns)."""
+    _gpu(proj, freqs, positions)
+    z, T = sizes, proj.shape[0]
+    _need(z.groups == z.heads, "every head has a key and a query of its own")
+    _need(proj.dtype == torch.float32 and proj.dim() == 2 and proj.is_contiguous() and proj.shape[1] >= z.channels,
+          lambda: f"the projected rows must be contiguous float32 [tokens, >= {z.channels}]")
+    _check_step_vectors(T, positions=positions)
+    rot = 0 if freqs is None else 2 * freqs.shape[0]
+    _check_freqs(freqs, rot)
+    _need(rot <= z.state, "at most a head's dimensions turn")
+    mixed = torch.empty((T, z.row), dtype=out_dtype, device=proj.device)
+    _run("retention_prepare", library().ts_retention_prepare(_ptr(mixed), _code(out_dtype), _ptr(proj), proj.shape[1], _ptr(freqs), _ptr(positions), T,
+                                                             z.heads, z.vdim, z.vp, z.state, z.np, rot, _stream()))
+    return mixed
+
+
+DELTA_MAX_CHUNK_PLACES = 256     # of a key: longer ones walk token by token whatever the portion
+DELTA_CHUNKS_FROM = 24           # tokens of a request's portion from which it is worked in chunks (bfloat16 only)
+
+
+class DeltaRows:
+    """What `delta_prepare` makes of a step's projected rows for `delta_scan`: mixed rows [tokens, row] (v, k, q in the places of
+    `SsdSizes`: x, B, C), units float32 [tokens, 2 groups] (the factors that make k, then q, unit vectors; q's with
+    dim^(-1/2)), betas and logs float32 [tokens, heads]."""
+
+    __slots__ = ("mixed", "units", "betas", "logs")
+
+    def __init__(self, mixed: torch.Tensor, units: torch.Tensor, betas: torch.Tensor, logs: torch.Tensor) -> None:
+        self.mixed, self.units, self.betas, self.logs = mixed, units, betas, logs
+
+
+def delta_prepare(proj: torch.Tensor, conv_w: torch.Tensor, dt_bias: torch.Tensor, a_log: torch.Tensor, state: torch.Tensor, ctx,
+                  sizes: SsdSizes, out_dtype: torch.dtype) -> DeltaRows:
+    """From projected rows (float32 [tokens, >= projected + heads], gate | v | k | q | a | b leading) to the gated delta
+    rule's operands: v, k and q through the causal convolution and silu, as `out_dtype`; beta = sigmoid(b), log decay
+    -exp(a_log) softplus(a + dt_bias). conv_w float32 [taps, row] in the places of a mixed row (`SsdSizes.spread`). The rows
+    ahead of a request's first token of the step come from its slot of `state` (float32 [slots, >= matrix + kept], the
+    convolution's inputs behind S), where the step leaves its own last ones."""
+    _gpu(proj, conv_w, dt_bias, a_log, state)
+    T, z = proj.shape[0], sizes
+    _need(proj.dtype == torch.float32 and proj.dim() == 2 and proj.is_contiguous() and proj.shape[1] >= z.projected + z.heads,
+          lambda: f"the projected rows must be contiguous float32 [tokens, >= {z.projected + z.heads}]")
+    _need(conv_w.dtype == torch.float32 and conv_w.shape == (z.taps, z.row) and conv_w.is_contiguous(), lambda: f"conv_w must be float32 [{z.taps}, {z.row}]")
+    _check_head_vectors(z.heads, dt_bias, a_log)
+    _check_ssd_state(state, z)
+    _check_step_requests(ctx)
+    _need(ctx.num_tokens == T, "the projected rows are the step's")
+    rows = DeltaRows(torch.empty((T, z.row), dtype=out_dtype, device=proj.device),
+                     *(torch.empty((T, n), dtype=torch.float32, device=proj.device) for n in (2 * z.groups, z.heads, z.heads)))
+    kept = state.data_ptr() + 4 * z.matrix
+    # (a request's only token of the step moves its slot on by itself: nobody else reads it)
+    moves = z.taps > 1 and T == ctx.num_seqs and ctx.max_query_len == 1
+    _run("delta_prepare", library().ts_delta_prepare(
+        _ptr(rows.mixed), _code(out_dtype), _ptr(rows.units), _ptr(rows.betas), _ptr(rows.logs), _ptr(proj), proj.shape[1], _ptr(conv_w), kept,
+        state.stride(0), _ptr(dt_bias), _ptr(a_log), _ptr(ctx.cu_seqlens), _ptr(ctx.seq_of_token), _ptr(ctx.state_slots), T, z.heads, z.vdim,
+        z.vp, z.groups, z.state, z.np, z.taps, float(z.state) ** -0.5, int(moves), _stream()))
+    if z.taps > 1 and not moves:
+        _run("ssd_conv_keep", library().ts_ssd_conv_keep(
+            kept, state.stride(0), _ptr(proj), proj.shape[1], _ptr(ctx.cu_seqlens), _ptr(ctx.state_slots), ctx.num_seqs, z.heads, z.vdim, z.vp,
+            z.groups, z.state, z.np, z.taps, _stream()))
+    return rows
+
+
+def delta_scan(rows: DeltaRows, state: torch.Tensor, ctx, sizes: SsdSizes, chunks_from: int = DELTA_CHUNKS_FROM) -> torch.Tensor:
+    """The gated delta rule over a packed step: per head, with unit vectors k and q, S <- exp(log) S, u = beta (v - S^T k),
+    S <- S + k u^T, o = S^T q, each request from and to its slot of `state` (S as [heads, vp, np], a value column's places side
+    by side, at the start of the slot's row). Returns o float32 [tokens, heads vdim]. In bfloat16, requests that feed at least
+    `chunks_from` tokens are worked in chunks on the matrix cores; all others, and 32-bit rows always, token by token."""
+    z, mixed = sizes, rows.mixed
+    T = mixed.shape[0]
+    _gpu(mixed, rows.units, rows.betas, rows.logs, state)
+    _need(mixed.shape == (T, z.row) and mixed.is_contiguous(), lambda: f"the mixed rows must be contiguous [tokens, {z.row}]")
+    for t, n in ((rows.units, 2 * z.groups), (rows.betas, z.heads), (rows.logs, z.heads)):
+        _need(t.dtype == torch.float32 and t.shape == (T, n) and t.is_contiguous(), "units, betas and logs must be float32, a row per token")
+    _check_ssd_state(state, z)
+    _check_step_requests(ctx)
+    _need(ctx.num_tokens == T and chunks_from >= 1, "the mixed rows are the step's")
+    S, dev = ctx.num_seqs, mixed.device
+    out = torch.empty((T, z.inner), dtype=torch.float32, device=dev)
+    chunked = mixed.dtype == torch.bfloat16 and ctx.max_query_len >= chunks_from and z.np <= DELTA_MAX_CHUNK_PLACES
+    if chunked:
+        chunks, chunk_cu = _step_chunks(ctx, chunks_from, dev)
+        C, L = chunks.shape[0], SSD_CHUNK
+        tiles = torch.empty((2, C, z.heads, 2, L, L), dtype=torch.bfloat16, device=dev)
+        turned = torch.empty((C, z.groups * z.np + z.heads * z.vp, L), dtype=torch.bfloat16, device=dev)
+        scales = torch.empty((C * z.heads * (4 * L + 1),), dtype=torch.float32, device=dev)
+        _run("delta_chunks", library().ts_delta_chunks(
+            _ptr(out), _ptr(mixed), _ptr(rows.units), _ptr(rows.betas), _ptr(rows.logs), _ptr(state), state.stride(0), _ptr(chunks), _ptr(chunk_cu),
+            _ptr(ctx.state_slots), _ptr(tiles), tiles[1].data_ptr(), _ptr(turned), turned.data_ptr() + 2 * L * C * z.groups * z.np, _ptr(scales),
+            scales.data_ptr() + 4 * 4 * L * C * z.heads, C, S, z.heads, z.vdim, z.vp, z.groups, z.np, _stream()))
+        if _all_in_chunks(ctx, chunks_from):
+            return out
+    _run("delta_step", library().ts_delta_step(
+        _ptr(out), _ptr(mixed), _code(mixed.dtype), _ptr(rows.units), _ptr(rows.betas), _ptr(rows.logs), _ptr(state), state.stride(0),
+        _ptr(ctx.cu_seqlens), _ptr(ctx.state_slots), S, z.heads, z.vdim, z.vp, z.groups, z.np, chunks_from - 1 if chunked else 0, _stream()))
+    return out
+
+
+# ---- capped logits ----
+
+def soft_cap(x: torch.Tensor, cap: float) -> torch.Tensor:
+    """x = cap tanh(x / cap), in place on a contiguous float32 tensor; returns it."""
+    _gpu(x)
+    _need(x.dtype == torch.float32 and x.is_contiguous() and x.data_ptr() % 16 == 0 and cap > 0, "contiguous float32, a positive cap")
+    _run("soft_cap", library().ts_soft_cap(_ptr(x), float(cap), x.numel(), _stream()))
+    return x

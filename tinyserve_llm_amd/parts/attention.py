@@ -141,7 +141,7 @@ class GeneralAttention(Mixer):
                  position: str | None = None, scale: float | None = None, softcap: float = 0.0, sink: bool = False,
                  qk_norm_eps: float | None = None, v_norm_eps: float | None = None, window: int = 0, chunk: int = 0,
                  learned_sink: bool = False, projection_norm_eps: float | None = None, head_norm_eps: float | None = None,
-                 value_position: str | None = None, head_gate: bool = False) -> None:
+                 value_position: str | None = None, head_gate: bool = False, bias: bool = False) -> None:
         """Further options. `chunk` (instead of `window`): a position sees the keys of its own chunk of that many
         positions, chunks counted from position 0. `learned_sink`: exp(sink[h]), a learned number per head, in the
         softmax's denominator (instead of `sink`'s 1). `projection_norm_eps`: the whole q projection of a token (all
@@ -151,11 +151,13 @@ class GeneralAttention(Mixer):
         share (`q_norm`, `k_norm`), before the heads turn. `value_position` names a `rotary_frequencies` encoding over
         all of `value_dim`: the value at position j is turned by j before it is cached, and each head's output at position
         i is turned back by i. `head_gate`: each head's output (turned back) is multiplied by sigmoid(W_gate h)_head, one
-        number per head."""
+        number per head; without `value_position` W_gate's rows are the fused projection's last ones and the gate rides on
+        the attention kernels' way out. `bias`: q, k and v have biases (`qkv_bias`, 32-bit), added ahead of every norm; they
+        ride on the kernel that norms the whole projections (`projection_norm_eps`)."""
         if projection_norm_eps is not None and head_norm_eps is not None:
             raise ValueError("a norm over the whole q and k projections or over every head, not both")
-        if head_gate and value_position is None:
-            raise ValueError("the gate per head rides on the kernel that turns the heads' outputs back (value_position)")
+        if bias and projection_norm_eps is None:
+            raise ValueError("the biases ride on the kernel that norms the whole q and k projections (projection_norm_eps)")
         if chunk < 0 or window < 0 or (chunk and window):
             raise ValueError("a sliding window or chunks (both >= 0), not both")
         if sink and learned_sink:
@@ -173,8 +175,11 @@ class GeneralAttention(Mixer):
         self.softcap, self.sink, self.qk_norm_eps, self.v_norm_eps, self.window = softcap, sink, qk_norm_eps, v_norm_eps, window
         self.chunk, self.learned_sink, self.projection_norm_eps = chunk, learned_sink, projection_norm_eps
         self.head_norm_eps, self.value_position, self.head_gate = head_norm_eps, value_position, head_gate
+        self.has_bias = bias
+        self.gate_inside = head_gate and value_position is None      # the gate's rows lie behind q, k and v
         self.gate: torch.Tensor | None = None
         self.qkv: torch.Tensor | None = None
+        self.qkv_bias: torch.Tensor | None = None
         self.o: torch.Tensor | None = None
         self.q_norm: torch.Tensor | None = None
         self.k_norm: torch.Tensor | None = None
@@ -194,20 +199,34 @@ class GeneralAttention(Mixer):
     def v_size(self) -> int:
         return self.num_kv_heads * self.value_dim
 
+    @property
+    def projected(self) -> int:
+        """Rows of the fused projection: q, k, v, and the gate's where they lie there (rows of zeros then fill it up to a
+        multiple of eight: its result's rows start at 16-byte borders)."""
+        rows = self.q_size + self.k_size + self.v_size
+        return -(-(rows + self.num_heads) // 8) * 8 if self.gate_inside else rows
+
     def param_specs(self) -> dict[str, ParamSpec]:
-        specs = {"qkv": ParamSpec((self.q_size + self.k_size + self.v_size, self.hidden_size)),
+        specs = {"qkv": ParamSpec((self.projected, self.hidden_size)),
                  "o": ParamSpec((self.hidden_size, self.num_heads * self.value_dim))}
+        if self.has_bias:
+            specs["qkv_bias"] = ParamSpec((self.q_size + self.k_size + self.v_size,), "float32", init=(0.0, 0.1))
         if self.projection_norm_eps is not None:
             specs["q_norm"] = ParamSpec((self.q_size,), "float32", init=(1.0, 0.1))
             specs["k_norm"] = ParamSpec((self.k_size,), "float32", init=(1.0, 0.1))
         if self.head_norm_eps is not None:
             specs["q_norm"] = ParamSpec((self.head_dim,), "float32", init=(1.0, 0.1))
             specs["k_norm"] = ParamSpec((self.head_dim,), "float32", init=(1.0, 0.1))
-        if self.head_gate:
+        if self.head_gate and not self.gate_inside:
             specs["gate"] = ParamSpec((self.num_heads, self.hidden_size))
         if self.learned_sink:
             specs["sinks"] = ParamSpec((self.num_heads,), "float32", init=(0.0, 1.0))
         return specs
+
+    def bind(self, params) -> None:
+        super().bind(params)
+        if self.gate_inside:
+            self.qkv[self.q_size + self.k_size + self.v_size + self.num_heads:].zero_()
 
     def kv_spec(self) -> KVSpec:
         # (a chunk's keys lie within the last `chunk` positions: the cache may give back what lies before them)
@@ -222,9 +241,11 @@ class GeneralAttention(Mixer):
         enc = ctx.position_encodings[self.position] if self.position else None
         slots = ctx.slot_mapping[mem.space] if mem.store else None
         k_store, v_store = (mem.k_cache, mem.v_cache) if mem.store else (None, None)
+        gate_at = self.q_size + self.k_size + self.v_size
         qkv = linear(x, self.qkv, out_dtype=torch.float32, packed=self.qkv_packed)
         if self.projection_norm_eps is not None:         # in place, each over its whole stretch of the row
-            hip.segment_rmsnorm_pair(qkv, (0, self.q_size, self.q_norm), (self.q_size, self.k_size, self.k_norm), self.projection_norm_eps)
+            hip.segment_rmsnorm_pair(qkv, (0, self.q_size, self.q_norm), (self.q_size, self.k_size, self.k_norm), self.projection_norm_eps,
+                                     bias=self.qkv_bias, rest=(self.q_size + self.k_size, self.v_size) if self.has_bias else (0, 0))
         value_enc = ctx.position_encodings[self.value_position] if self.value_position else None
         if self.head_norm_eps is not None or value_enc is not None:      # in place: the heads' norms, the values' turn
             hip.qkv_prepare(qkv, ctx.positions, self.num_heads, self.num_kv_heads, self.head_dim, self.value_dim,
@@ -237,7 +258,7 @@ class GeneralAttention(Mixer):
                            interleaved=getattr(enc, "interleaved", True), qk_norm_eps=self.qk_norm_eps,
                            v_norm_eps=self.v_norm_eps, amplitude=getattr(enc, "amplitude", 1.0))
         o = hip.paged_attention(q, mem.k_cache, mem.v_cache, ctx, mem.space, self.scale, self.window, softcap=self.softcap,
-                                sink=self.sink, sinks=self.sinks, chunk_mask=self.chunk)
+                                sink=self.sink, sinks=self.sinks, chunk_mask=self.chunk, gate=qkv[:, gate_at:gate_at + self.num_heads] if self.gate_inside else None)
         if value_enc is not None:                         # each head's sum turned back by its own position, then its gate
             gate = linear(x, self.gate, out_dtype=torch.float32) if self.head_gate else None
             hip.rotate_heads(o, o, value_enc.frequencies(), 1.0, ctx.positions, interleaved=value_enc.interleaved, back=True, gate=gate)

@@ -193,6 +193,28 @@ def pre_norm_stream_block(layer: Layer, hidden, residual, ctx: StepContext, mem:
     return ResidualStream(x, layer.feed_forward.forward(h, ctx)), None
 
 
+@register("block", "post_norm_stream")
+@uses_norms("norm1")
+@keeps_stream
+def post_norm_stream_block(layer: Layer, hidden, residual, ctx: StepContext, mem: LayerMemory):
+    """x <- x + norm1(mixer(x)), then x <- x + norm2(feed_forward(x)): the parts read the stream itself, and what they make
+    is normed on its way into it ("norm2" only where the layer has a feed-forward). The stream is 32-bit; each sum is left
+    pending in it with the norm the branch's rows still have to pass, so that whoever takes the stream next does norm and
+    sum in one kernel, which also leaves the rows as the next projection's operand."""
+    from tinyserve_llm_amd.parts.stream import ResidualStream
+    if not isinstance(hidden, ResidualStream) or residual is not None:
+        raise TypeError("this arrangement runs on a 32-bit residual stream (ModelSpec.residual_dtype = 'float32')")
+    norms = layer.norms
+    x, rows = hidden.rows_as(norms["norm1"].weight.dtype)
+    stream = ResidualStream(x, layer.mixer.forward(rows, ctx, mem), post=norms["norm1"])
+    if "norm2" not in norms:
+        if layer.feed_forward.forward(None, ctx) is not None:
+            raise KeyError("a layer with a feed-forward names the norm 'norm2'")
+        return stream, None
+    x, rows = stream.rows_as(norms["norm2"].weight.dtype)
+    return ResidualStream(x, layer.feed_forward.forward(rows, ctx), post=norms["norm2"]), None
+
+
 @register("block", "sandwich_scaled")
 @uses_norms("norm1", "norm1b", "scale1")
 @keeps_stream

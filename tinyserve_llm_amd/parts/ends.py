@@ -67,11 +67,16 @@ class TableEmbedding(Embedding):
 
 @register("head", "projection")
 class ProjectionHead(Head):
-    """float32 logits = rows · Wᵀ with W [vocab, hidden], its own or the embedding's."""
+    """float32 logits = rows · Wᵀ with W [vocab, hidden], its own or the embedding's; with `softcap` > 0 they leave as
+    softcap tanh(logits / softcap)."""
 
     graph_safe = True
 
-    def __init__(self, vocab_size: int, hidden_size: int, tied: bool = False, init: tuple[float, float] = (0.0, 0.02)) -> None:
+    def __init__(self, vocab_size: int, hidden_size: int, tied: bool = False, init: tuple[float, float] = (0.0, 0.02),
+                 softcap: float = 0.0) -> None:
+        if softcap < 0:
+            raise ValueError(f"softcap {softcap}: positive, or 0 for none")
+        self.softcap = float(softcap)
         self.vocab_size, self.hidden_size, self.tied, self.init = vocab_size, hidden_size, tied, tuple(init)
         self.weight: torch.Tensor | None = None
         self.weight_packed = None                # `streaming_copy` of the weight, if the model keeps them
@@ -90,4 +95,5 @@ class ProjectionHead(Head):
         return 0 if self.weight_packed is None else self.weight_packed.nbytes()
 
     def forward(self, rows: torch.Tensor) -> torch.Tensor:
-        return linear(rows, self.weight, out_dtype=torch.float32, packed=self.weight_packed)
+        logits = linear(rows, self.weight, out_dtype=torch.float32, packed=self.weight_packed)
+        return hip.soft_cap(logits, self.softcap) if self.softcap else logits

@@ -24,14 +24,20 @@ class RoutedExperts(FeedForward):
     over all the router's outputs instead of sigmoids. `identity`: the router has that many more outputs than there
     are experts with matrices; they stand for experts that hand their input through (times the weight). `shared_gate`:
     the shared expert's output is multiplied by sigmoid(w_sg . h), one number per token; w_sg is the router's last
-    row, so that its logit is 32-bit like the others."""
+    row, so that its logit is 32-bit like the others. `groups` = (count, keep): the experts, identity experts included,
+    form `count` equal groups of neighbours, and only those of the `keep` groups with the largest best s + correction can be
+    chosen."""
 
     graph_safe = True
 
     def __init__(self, hidden_size: int, num_experts: int, top: int, intermediate_size: int, limit: float = 0.0,
                  slope: float = 1.702, up_shift: float = 1.0, router_scale: float = 1.0, normalize: bool = True,
                  correction: bool = True, shared: dict | None = None, scoring: str = "sigmoid", identity: int = 0,
-                 shared_gate: bool = False) -> None:
+                 shared_gate: bool = False, groups: tuple[int, int] = (1, 1)) -> None:
+        count, keep = groups
+        if not 1 <= keep <= count <= hip.MOE_MAX_GROUPS or (num_experts + identity) % count or top > keep * ((num_experts + identity) // count):
+            raise ValueError(f"groups {groups}: {num_experts + identity} experts in equal groups, of which those kept hold at least {top}")
+        self.groups = (int(count), int(keep))
         if scoring not in ("sigmoid", "softmax_all") or identity < 0 or (shared_gate and shared is None):
             raise ValueError("scoring 'sigmoid' or 'softmax_all'; identity >= 0; a gate on the shared expert needs one")
         if top > num_experts + identity or num_experts + identity > hip.MOE_MAX_EXPERTS:
@@ -74,7 +80,7 @@ class RoutedExperts(FeedForward):
 
     def forward(self, x: torch.Tensor, ctx: StepContext) -> torch.Tensor:
         routed = hip.moe_route(x, self.router, self.correction, self.top, self.router_scale, self.normalize,
-                               softmax_all=self.scoring == "softmax_all", extras=int(self.shared_gate))
+                               softmax_all=self.scoring == "softmax_all", extras=int(self.shared_gate), groups=self.groups)
         experts, weights = routed[0], routed[1]
         tile_rows = hip.moe_tile_rows(experts.numel(), self.num_experts, x.dtype, (self.hidden_size, self.intermediate_size))
         grouped = hip.moe_group(experts, self.num_experts, tile_rows)

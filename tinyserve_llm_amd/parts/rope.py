@@ -71,8 +71,9 @@ class RotaryFrequencies(PositionEncoding):
 
     graph_safe = True
 
-    def __init__(self, rotary_dim: int, theta: float, interleaved: bool = True, ramp: dict | None = None, bands: dict | None = None) -> None:
-        """`ramp` (factor s, original length L, fast, slow): frequencies are slowed down by s along a ramp over
+    def __init__(self, rotary_dim: int, theta: float, interleaved: bool = True, ramp: dict | None = None, bands: dict | None = None,
+                 divide: float = 1.0) -> None:
+        """`divide`: every f_i is divided by it (linear scaling of the positions). `ramp` (factor s, original length L, fast, slow): frequencies are slowed down by s along a ramp over
         the pairs: with d(t) = rotary_dim ln(L / (2 pi t)) / (2 ln theta), lo = max(floor d(fast), 0),
         hi = min(ceil d(slow), rotary_dim - 1) and r_i = clamp((i - lo) / max(hi - lo, 0.001), 0, 1), pair i
         turns with f_i / s * r_i + f_i (1 - r_i), and cosine and sine are multiplied by `amplitude` =
@@ -81,6 +82,9 @@ class RotaryFrequencies(PositionEncoding):
         f / s, those between (1 - m) f / s + m f with m = (L / l - low) / (high - low); no amplitude."""
         if ramp and bands:
             raise ValueError("frequencies slow down along a ramp or in bands, not both")
+        if not divide > 0 or (divide != 1.0 and (ramp or bands)):
+            raise ValueError("frequencies are divided by a positive number, and then not along a ramp or in bands too")
+        self.divide = float(divide)
         if rotary_dim % 2 or rotary_dim < 0:
             raise ValueError(f"rotary_dim {rotary_dim}: an even number of dimensions turns")
         self.rotary_dim, self.theta, self.interleaved = rotary_dim, float(theta), interleaved
@@ -105,7 +109,7 @@ class RotaryFrequencies(PositionEncoding):
             between = (1.0 - mix) * f / b["factor"] + mix * f
             return torch.where(turns > b["high"], f, torch.where(turns < b["low"], f / b["factor"], between))
         if self.ramp is None:
-            return f
+            return f / self.divide
         r = self.ramp
 
         def crossing(turns: float) -> float:

@@ -59,7 +59,8 @@ class ResidualStream:
             return self.settle()[0], self.x
         if hasattr(self.post, "weight32"):
             return self.x, self._apply_post(out_dtype=dtype)
-        raise TypeError("the stream's rows leave in another type on the way out of an RMS norm's sum")
+        x = self.settle()[0]
+        return x, hip.bias_activation(x, None, "none", dtype)
 
     def take(self, norm=None, rows: torch.Tensor | None = None, out_dtype: torch.dtype = torch.float32):
         """Does the pending sum and returns (x, norm(x)) (norm(x) of the picked `rows` only if given; None
