@@ -193,6 +193,19 @@ def choose(z: torch.Tensor, correction: torch.Tensor, top: int, groups: int, kee
     return chosen, [float(s[e]) for e in chosen]
 
 
+def choice_margin(z: torch.Tensor, correction: torch.Tensor, top: int, groups: int, keep: int) -> float:
+    """By how much of its score (the larger of the two scores) the weakest thing chosen is ahead of the strongest one left
+    out, expert or group, whichever is closer: a small number is a choice that rounding may turn round."""
+    s = torch.softmax(z, dim=-1)
+    choice = s + correction
+    size = z.shape[0] // groups
+    lead = [max(range(a * size, (a + 1) * size), key=lambda e: float(choice[e])) for a in range(groups)]
+    lead.sort(key=lambda e: -float(choice[e]))
+    allowed = sorted((e for a in lead[:keep] for e in range(a // size * size, (a // size + 1) * size)), key=lambda e: -float(choice[e]))
+    pairs = ([(lead[keep - 1], lead[keep])] if keep < groups else []) + ([(allowed[top - 1], allowed[top])] if top < len(allowed) else [])
+    return min((float(choice[a] - choice[b]) / float(max(s[a], s[b])) for a, b in pairs), default=math.inf)
+
+
 def experts_unit(h: torch.Tensor, W: dict, c: dict) -> torch.Tensor:
     router = c["router"]
     real, groups = int(router["experts"]), router.get("groups") or {"count": 1, "keep": 1}
@@ -214,6 +227,7 @@ class PlainKufolorn:
         self.memory: list[dict] = []
         self.fed = 0
         self.after_layers: list[torch.Tensor] = []      # the residual stream after every layer, of the last call
+        self.margin = math.inf                          # the closest call of any router, of the last call (`choice_margin`)
 
     @classmethod
     def from_folder(cls, folder: str, dtype: torch.dtype = torch.float64) -> "PlainKufolorn":
@@ -247,12 +261,16 @@ class PlainKufolorn:
         positions = torch.arange(self.fed, self.fed + len(tokens))
         self.fed += len(tokens)
         x = self.w["embed"][torch.tensor(tokens)]
-        self.after_layers = []
+        self.after_layers, self.margin = [], math.inf
         for i, layer in enumerate(c["layers"]):
             x = x + layer_norm(self.mixer(i, x, positions, self.memory[i]), self.w[f"l{i}.norm1"], eps)
             mlp = layer.get("mlp")
             if mlp is not None:
                 W = self._sub(f"l{i}.mlp.")
+                if mlp["kind"] == "moe":
+                    r = mlp["router"]
+                    g = r.get("groups") or {"count": 1, "keep": 1}
+                    self.margin = min([self.margin] + [choice_margin(W["router"] @ h, W["correction"], r["top"], g["count"], g["keep"]) for h in x])
                 y = dense_unit(x, W) if mlp["kind"] == "dense" else experts_unit(x, W, mlp)
                 x = x + layer_norm(y, self.w[f"l{i}.norm2"], eps)
             self.after_layers.append(x.clone())

@@ -25,7 +25,7 @@ class KufolornRotation:
             return cls(0, 1.0)
         scaling = raw.get("scaling")
         c = cls(dims=int(_need(raw, "dims", where)), base=float(_need(raw, "base", where)),
-                factor=float(_need(scaling, "factor", where + ".scaling")) if scaling else 1.0)
+                factor=1.0 if scaling is None else float(_need(scaling, "factor", where + ".scaling")))
         if c.dims < 0 or c.dims % 2 or not c.base > 0 or not c.factor > 0:
             raise ConfigError(f"{where}: an even number of dims, a positive base and a positive scaling.factor")
         return c
@@ -171,7 +171,7 @@ def _mlp(raw: Mapping[str, Any] | None, where: str) -> "KufolornDense | Kufolorn
     if kind == "moe":
         router, expert = _need(raw, "router", where), _need(raw, "expert", where)
         groups = router.get("groups")
-        count, keep = (int(_need(groups, k, where + ".router.groups")) for k in ("count", "keep")) if groups else (1, 1)
+        count, keep = (int(_need(groups, k, where + ".router.groups")) for k in ("count", "keep")) if groups is not None else (1, 1)
         e = KufolornExperts(experts=int(_need(router, "experts", where + ".router")), identity=int(router.get("identity") or 0),
                             top=int(_need(router, "top", where + ".router")), ff=int(_need(expert, "ff", where + ".expert")),
                             limit=float(_need(expert, "limit", where + ".expert")), groups=count, keep=keep)
