@@ -52,6 +52,12 @@ windowed attention and attention through a latent with learned sinks and a gate 
 each pass behind a projection of the stream and the embedded tokens) beside the Bafarax decoder, the closest of the
 engine's models, at equal layer sizes and as many runs of a layer, in the same way. One JSON line.
 
+    python bench.py --kufolorn [--shape 1b|3b] [--layers L] [--kernels-only]
+
+measures the Kufolorn decoder (norms on the way into a 32-bit stream whose rows the sublayers read as they are; a gated delta
+rule in turn with attention beside retention; gelu-gated and routed feed-forwards, experts chosen inside groups; capped
+logits) beside the Tegolix decoder, the closest of the engine's models, at equal layer sizes, in the same way. One JSON line.
+
     python bench.py --scenario requests-3b | chunked-8b [--layers L]
 
 runs a whole workload through `LLM.generate` instead and prints one JSON line of its own: many
@@ -1220,6 +1226,195 @@ def morulix(args) -> int:
     return 0
 
 
+def kufolorn_design(shape: str, layers: int | None):
+    """The Kufolorn configuration that `--kufolorn` measures at the layer sizes of `shape`, and those sizes by name."""
+    from tinyserve_llm_amd.config.kufolorn import (KufolornAttention, KufolornConfig, KufolornDelta, KufolornDense, KufolornExperts, KufolornLayer,
+                                                   KufolornParallel, KufolornRetention, KufolornRotation)
+    sizes = SHAPES[shape]
+    sh = sizes["shape"]
+    layers = layers or sizes["layers_full"]
+    hidden, nh, nkv, hd, inter, vocab = (sh["hidden_size"], sh["num_attention_heads"], sh["num_key_value_heads"], sh["head_dim"],
+                                         sh["intermediate_size"], sh["vocab_size"])
+    # a delta rule of heads of 128, the values together twice as wide as the model and two heads to a key; beside attention of
+    # the shape's heads over every position before, retention of heads of 128 as wide as the model; 16 experts of a quarter of
+    # the dense width and two identity experts in three groups of which two are kept, of which a token uses 4
+    dd, taps, experts, identity, groups, keep, top, eff = 128, 4, 16, 2, 3, 2, 4, inter // 4
+    dg, rh = hidden // dd, hidden // dd
+    dh = 2 * dg
+    decay = tuple(1.0 - 2.0 ** (-5.0 - 6.0 * i / max(1, rh - 1)) for i in range(rh))
+    delta = KufolornDelta(heads=dh, kv_heads=dg, dim=dd, vdim=dd, conv=taps)
+    left = KufolornAttention(heads=nh, kv_heads=nkv, dim=hd, vdim=hd, scale=hd ** -0.5, rot=KufolornRotation(hd, 250000.0, 4.0))
+    right = KufolornRetention(heads=rh, dim=dd, vdim=dd, decay=decay, rot=KufolornRotation(dd, 10000.0))
+    par = KufolornParallel(left, right, left_scale=0.8, right_scale=0.9)
+    moe = KufolornExperts(experts=experts, identity=identity, top=top, ff=eff, limit=7.0, groups=groups, keep=keep)
+    cycle = (("delta", delta, KufolornDense(inter)), ("parallel", par, moe)) * 2
+    kuf = KufolornConfig(vocab=vocab, width=hidden, norm_eps=1e-6, logit_softcap=30.0, layers=tuple(KufolornLayer(*cycle[i % 4]) for i in range(layers)))
+    return kuf, dict(layers=layers, delta_heads=dh, delta_groups=dg, delta_dim=dd, conv_taps=taps, retention_heads=rh, retention_dim=dd, experts=experts,
+                     identity=identity, groups=groups, keep=keep, top=top, eff=eff)
+
+
+def kufolorn(args) -> int:
+    """The Kufolorn decoder beside the Tegolix decoder (the engine's closest design: pairs of attention and a recurrence,
+    recurrences of their own in turn with them, norms on the way into a 32-bit stream, a softmax router with identity experts)
+    at the layer sizes of `--shape`: whole-engine throughput, and the like kernels of the two side by side (the state-space
+    mixer's convolution and recurrence beside them). One JSON line."""
+    import torch
+
+    from tinyserve_llm_amd.ops import hip
+
+    teg, t = tegolix_design(args.shape, args.layers)
+    kuf, z = kufolorn_design(args.shape, args.layers)
+    _, m = morulix_design(args.shape, args.layers)
+    sh = SHAPES[args.shape]["shape"]
+    hidden, nh, nkv, hd, inter, vocab = (sh["hidden_size"], sh["num_attention_heads"], sh["num_key_value_heads"], sh["head_dim"],
+                                         sh["intermediate_size"], sh["vocab_size"])
+    window, gh, gd, gv, rh, rd = t["window"], t["gh"], t["gd"], t["gv"], t["rh"], t["rd"]
+    prompt_len = args.context
+    bench = DesignBench(vocab, prompt_len)
+    timed, context = bench.timed, bench.context
+    bf = torch.bfloat16
+
+    def kernel_pairs() -> dict:
+        pairs = {}
+        pool_page = 32
+        peaks = hip.measure_peaks()
+        read_peak, mfma_peak, vector_peak = peaks["read_GBps"] * 1e9, peaks["mfma_bf16_TFLOPs"] * 1e12, PEAK_FLOPS["fp32"]
+        sinks = torch.randn(nh, device="cuda")
+        delta = hip.SsdSizes(z["delta_heads"], z["delta_dim"], z["delta_groups"], z["delta_dim"], z["conv_taps"])
+        ret = hip.SsdSizes(z["retention_heads"], z["retention_dim"], z["retention_heads"], z["retention_dim"], 1)
+        ssd = hip.SsdSizes(m["ssm_heads"], m["ssm_vdim"], m["ssm_groups"], m["ssm_state"], m["conv_taps"])
+        for label, starts, counts in (("prompt portion", [0], [prompt_len]), ("decoded tokens, batch 64", [prompt_len + 511] * 64, [1] * 64),
+                                      ("decoded token", [prompt_len + 511], [1])):
+            ctx, slots, pages = context(starts, counts, pool_page)
+            T, prompt, R = ctx.num_tokens, ctx.num_tokens > 64, len(starts)
+            of_peak = lambda flops, nbytes, us: ({"frac_of_mfma": flops / us * 1e6 / mfma_peak} if prompt else
+                                                 {"frac_of_read": nbytes / us * 1e6 / read_peak})
+
+            def entry(name, **both):
+                """name_us, its bytes (and operations) and their shares of the peaks, for each side: side = (us, bytes[, flops])."""
+                out = {}
+                for side, (us, nbytes, *flops) in both.items():
+                    out.update({f"{side}_us": us, f"{side}_bytes": nbytes, f"{side}_frac_of_read": nbytes / us * 1e6 / read_peak})
+                    if flops:
+                        out.update({f"{side}_flops": flops[0], f"{side}_frac_of_fp32_vector": flops[0] / us * 1e6 / vector_peak})
+                pairs[f"{name}, {label}"] = out
+            k = torch.randn(pages, nkv, pool_page, hd, device="cuda").to(bf).permute(0, 2, 1, 3)
+            v = torch.randn(pages, nkv, hd, pool_page, device="cuda").to(bf).permute(0, 3, 1, 2)
+            q = torch.randn(T, nh, hd, device="cuda").to(bf)
+            spans = list(zip(starts, counts))
+            seen_w = sum(min(p + 1, window) for s0, n in spans for p in range(s0, s0 + n))
+            seen_a = sum(p + 1 for s0, n in spans for p in range(s0, s0 + n))
+            gate = torch.randn(T, nh, device="cuda")
+            # attention over every position before with sinks and a gate per head, against a window with capped scores
+            us_k = timed(lambda: hip.paged_attention(q, k, v, ctx, 0, hd ** -0.5, sinks=sinks, gate=gate))
+            us_t = timed(lambda: hip.paged_attention(q, k, v, ctx, 0, hd ** -0.5, window, softcap=30.0))
+            pairs[f"attention, {label}"] = {
+                "kufolorn_us": us_k, "tegolix_us": us_t, "kufolorn_keys": seen_a, "tegolix_keys": seen_w,
+                "kufolorn": of_peak(4 * nh * hd * seen_a, seen_a * 2 * nkv * hd * 2, us_k),
+                "tegolix": of_peak(4 * nh * hd * seen_w, seen_w * 2 * nkv * hd * 2, us_t)}
+            # between projection and cache (Tegolix: and the heads turned back and gated behind attention)
+            qkv_row = (nh + 2 * nkv) * hd
+            wide = -(-(qkv_row + nh) // 8) * 8
+            qkv32, qkvg32 = torch.randn(T, qkv_row, device="cuda"), torch.randn(T, wide, device="cuda")
+            nw, qw, kw, bias = (torch.ones(n, device="cuda") for n in (hd, nh * hd, nkv * hd, qkv_row))
+            rfreqs, hfreqs = torch.rand(hd // 2, dtype=torch.float64, device="cuda"), torch.rand(hd // 4, dtype=torch.float64, device="cuda")
+            o16 = torch.randn(T, nh, hd, device="cuda").to(bf)
+
+            def kuf_finish():
+                hip.segment_rmsnorm_pair(qkvg32, (0, nh * hd, qw), (nh * hd, nkv * hd, kw), 1e-6, bias=bias, rest=((nh + nkv) * hd, nkv * hd))
+                return hip.qkv_finish(qkvg32, rfreqs, ctx.positions, slots, k, v, nh, nkv, hd, hd, bf, interleaved=False)
+
+            def teg_finish():
+                hip.qkv_prepare(qkv32, ctx.positions, nh, nkv, hd, hd, q_weight=nw, k_weight=nw, eps=1e-6, value_freqs=rfreqs)
+                out = hip.qkv_finish(qkv32, hfreqs, ctx.positions, slots, k, v, nh, nkv, hd, hd, bf, interleaved=False, amplitude=1.2)
+                hip.rotate_heads(o16, o16, rfreqs, 1.0, ctx.positions, interleaved=False, back=True, gate=gate)
+                return out
+            entry("between projection and cache", kufolorn=(timed(kuf_finish), T * qkv_row * (4 + 4 + 4 + 2)),
+                  tegolix=(timed(teg_finish), T * (qkv_row * (4 + 4 + 4 + 2) + nh * hd * 4)))
+            # the branch's norm and the stream's sum, the rows out as they are; against a scale and a norm on the way out as well
+            x32, a32, w32 = torch.randn(T, hidden, device="cuda"), torch.randn(T, hidden, device="cuda"), torch.ones(hidden, device="cuda")
+            entry("stream sum and norm", kufolorn=(timed(lambda: hip.stream_post_norm(x32, a32, w32, None, 1e-6, None, 0.0, bf)), T * hidden * (3 * 4 + 2)),
+                  tegolix=(timed(lambda: hip.stream_post_norm(x32, a32, w32, w32, 1e-6, w32, 1e-6, bf)), T * hidden * (3 * 4 + 2)))
+            entry("two sides' sum", kufolorn=(timed(lambda: hip.scaled_sum(x32, 0.8, a32, 0.9)), T * hidden * 12))
+            # the unit of the dense feed-forward, the router, the logits' cap
+            sums = torch.randn(T, 2 * inter, device="cuda")
+            entry("gated unit", kufolorn=(timed(lambda: hip.capped_glu(sums, 0.0, 1.0, 0.0, bf, activation="gelu_tanh")), T * inter * 10),
+                  tegolix=(timed(lambda: hip.capped_glu(sums, 0.0, 1.0, 0.0, bf, activation="relu")), T * inter * 10))
+            h16 = torch.randn(T, hidden, device="cuda").to(bf)
+            outputs = z["experts"] + z["identity"]
+            router, corr = torch.randn(outputs + 1, hidden, device="cuda") * 0.02, torch.zeros(outputs, device="cuda")
+            rbytes = T * hidden * 2 + outputs * hidden * 4
+            entry("router", kufolorn=(timed(lambda: hip.moe_route(h16, router[:outputs], corr, z["top"], 1.0, False, softmax_all=True, groups=(z["groups"], z["keep"]))), rbytes),
+                  tegolix=(timed(lambda: hip.moe_route(h16, router, corr, z["top"], 1.0, False, softmax_all=True, extras=1)), rbytes))
+            logits = torch.randn(min(T, 64), vocab, device="cuda")
+            entry("capped logits", kufolorn=(timed(lambda: hip.soft_cap(logits, 30.0)), logits.numel() * 8))
+            # the recurrences and what lies around them: delta rule and retention, against gated linear attention, the recurrence
+            # with token shift, and the state-space mixer
+            flops = lambda sizes, n: 2 * n * T * sizes.heads * sizes.vdim * sizes.state
+            dproj = torch.randn(T, -(-(delta.projected + delta.heads) // 8) * 8, device="cuda")
+            dconv = torch.randn(delta.taps, delta.row, device="cuda") * 0.4
+            dtb, alog = torch.full((delta.heads,), -3.0, device="cuda"), torch.zeros(delta.heads, device="cuda")
+            dstate = torch.zeros(R, delta.matrix + delta.kept, device="cuda")
+            dprep = lambda: hip.delta_prepare(dproj, dconv, dtb, alog, dstate, ctx, delta, bf)
+            rows = dprep()
+            o = hip.delta_scan(rows, dstate, ctx, delta)
+            us_dp, us_ds = timed(dprep), timed(lambda: hip.delta_scan(rows, dstate, ctx, delta))
+            dw = torch.ones(delta.vdim, device="cuda")
+            us_dn = timed(lambda: hip.mlstm_finish(o, dw, dproj[:, :delta.inner], delta.heads, delta.vdim, 1e-6, bf, silu_gate=True))
+            rproj = torch.randn(T, ret.channels + ret.inner, device="cuda")
+            pfreqs = torch.rand(ret.state // 2, dtype=torch.float64, device="cuda")
+            keeps = torch.tensor(kuf.layers[1].mixer.right.decay, device="cuda")
+            rlogs, rsteps = torch.log(keeps), torch.full((ret.heads,), ret.state ** -0.5, device="cuda")
+            rstate = torch.zeros(R, ret.matrix, device="cuda")
+            rprep = lambda: hip.retention_prepare(rproj, pfreqs, ctx.positions, ret, bf)
+            mixed = rprep()
+            ro = hip.ssd_scan(mixed, rsteps, rlogs, None, rstate, ctx, ret, keeps=keeps)
+            us_rp, us_rs = timed(rprep), timed(lambda: hip.ssd_scan(mixed, rsteps, rlogs, None, rstate, ctx, ret, keeps=keeps))
+            us_rn = timed(lambda: hip.mlstm_finish(ro, None, rproj[:, ret.channels:], ret.heads, ret.vdim, 1e-6, bf, silu_gate=True))
+            K, V = gh * gd, gh * gv
+            gproj = torch.randn(T, 2 * K + 2 * V, device="cuda")
+            gz, gbias, gnorm = torch.randn(T, K, device="cuda"), torch.full((K,), 3.0, device="cuda"), torch.ones(gv, device="cuda")
+            gstate = torch.zeros(R, K * gv, device="cuda")
+            gla = lambda: hip.decay_scan(gproj[:, :K], gproj[:, K:2 * K], gproj[:, 2 * K:2 * K + V], gz, gbias, gstate, ctx.cu_seqlens, ctx.state_slots, gh, gd, gv,
+                                         form="sigmoid_root", tau=16.0, q_scale=gd ** -0.5, longest=max(counts))
+            go = gla()
+            us_g = timed(gla)
+            us_gn = timed(lambda: hip.mlstm_finish(go, gnorm, gproj[:, 2 * K + V:], gh, gv, 1e-6, bf, silu_gate=True))
+            sr, sk, sv, szz = (torch.randn(T, rh * rd, device="cuda") for _ in range(4))
+            sbias, sbonus = torch.full((rh * rd,), -3.0, device="cuda"), torch.randn(rh, rd, device="cuda")
+            sstate = torch.zeros(R, rh * rd * rd, device="cuda")
+            us_sh = timed(lambda: hip.decay_scan(sr, sk, sv, szz, sbias, sstate, ctx.cu_seqlens, ctx.state_slots, rh, rd, rd, form="double_exponent", bonus=sbonus, longest=max(counts)))
+            mproj = torch.randn(T, -(-ssd.projected // 8) * 8, device="cuda")
+            mconv, mcb = torch.randn(ssd.taps, ssd.row, device="cuda") * 0.4, torch.zeros(ssd.row, device="cuda")
+            mdt, mal, mskip = torch.full((ssd.heads,), -3.0, device="cuda"), torch.zeros(ssd.heads, device="cuda"), torch.ones(ssd.heads, device="cuda")
+            mstate = torch.zeros(R, ssd.matrix + ssd.kept, device="cuda")
+            mprep = lambda: hip.ssd_prepare(mproj, mconv, mcb, mdt, mal, mstate, ctx, ssd, bf)
+            mrows = mprep()
+            us_mp, us_ms = timed(mprep), timed(lambda: hip.ssd_scan(*mrows, mskip, mstate, ctx, ssd))
+            scan_bytes = lambda sizes, extra: T * (sizes.row * 2 + sizes.heads * extra + sizes.inner * 4) + 2 * R * sizes.matrix * 4
+            conv_bytes = lambda sizes, extra: T * (sizes.channels * (4 + 2) + extra) + 2 * R * sizes.kept * 4
+            entry("recurrence, the scan", kufolorn_delta=(us_ds, scan_bytes(delta, 8) + T * delta.groups * 8, flops(delta, 3)),
+                  kufolorn_retention=(us_rs, scan_bytes(ret, 0), flops(ret, 2)),
+                  tegolix_gla=(us_g, T * (3 * K + 2 * V) * 4 + 2 * R * gstate.shape[1] * 4, 4 * T * gh * gd * gv),
+                  tegolix_shifted=(us_sh, T * 5 * rh * rd * 4 + 2 * R * sstate.shape[1] * 4, 4 * T * rh * rd * rd),
+                  morulix_state_space=(us_ms, scan_bytes(ssd, 8), flops(ssd, 2)))
+            entry("recurrence, ahead of the scan", kufolorn_delta=(us_dp, conv_bytes(delta, delta.heads * 16 + delta.groups * 8)),
+                  kufolorn_retention=(us_rp, T * ret.channels * 6), morulix_state_space=(us_mp, conv_bytes(ssd, ssd.heads * 12)))
+            entry("recurrence, norm and gate behind the scan", kufolorn_delta=(us_dn, T * delta.inner * 10), kufolorn_retention=(us_rn, T * ret.inner * 10),
+                  tegolix_gla=(us_gn, T * V * 10))
+        pairs["peaks"] = {"read_GBps": read_peak / 1e9, "mfma_bf16_TFLOPs": mfma_peak / 1e12, "fp32_vector_TFLOPs_published": vector_peak / 1e12}
+        return pairs
+
+    record = {"designs": {} if args.kernels_only else {"tegolix": bench.whole_engine(teg), "kufolorn": bench.whole_engine(kuf)},
+              "kernels": kernel_pairs(),
+              "config": {"shape": args.shape, "hidden": hidden, "heads": nh, "kv_heads": nkv, "head_dim": hd, "kufolorn": z, "tegolix": t,
+                         "kufolorn_layers": "in turn: a gated delta rule with a dense feed-forward of the shape's width, attention over every position "
+                                            "before beside retention, with experts",
+                         "vocab": vocab, "context": prompt_len, "dtype": "bf16", "data": "synthetic uniform token ids, random weights"}}
+    print(json.dumps(record))
+    return 0
+
+
 def kernel_classes(llm, config, batch: int, reps: int = 5) -> dict:
     """Times one decode step's kernels by class. An eager step (no graph) is run once with every
     launch of the engine's kernel module noted down with its operands; then each class's launches
@@ -1357,7 +1552,9 @@ def main() -> int:
                     help="the Tegolix decoder beside the Bafarax decoder at the layer sizes of --shape: throughput and like kernels")
     ap.add_argument("--morulix", action="store_true",
                     help="the Morulix decoder beside the Bafarax decoder at the layer sizes of --shape: throughput and like kernels")
-    ap.add_argument("--kernels-only", action="store_true", help="with --bafarax, --tegolix or --morulix: the kernels side by side, no whole-engine runs")
+    ap.add_argument("--kufolorn", action="store_true",
+                    help="the Kufolorn decoder beside the Tegolix decoder at the layer sizes of --shape: throughput and like kernels")
+    ap.add_argument("--kernels-only", action="store_true", help="with --bafarax, --tegolix, --morulix or --kufolorn: the kernels side by side, no whole-engine runs")
     ap.add_argument("--kernel-classes", action="store_true",
                     help="time one decode step's kernels class by class (bytes, microseconds, GB/s) and exit")
     ap.add_argument("--peaks", action="store_true",
@@ -1391,6 +1588,8 @@ def main() -> int:
         return tegolix(args)
     if args.morulix:
         return morulix(args)
+    if args.kufolorn:
+        return kufolorn(args)
     sizes = SHAPES[args.shape]
     full_layers = sizes["layers_full"]
     args.layers = args.layers or full_layers

@@ -631,7 +631,8 @@ def test_a_whole_delta_mixer(dtype, layer):
 # ---- whole models through trace replay ---------------------------------------------------------------
 
 LENGTHS = {"P": [1, 23, 97, 200], "Q": [1, 30, 75, 150], "R": [2, 19, 66, 131], "S": [1, 40, 140], "T": [1, 29, 110]}
-TOL = {"float32": 5e-5, "bfloat16": 6e-2}       # of the spread of the oracle's logits (a head whose read-out is nearly nothing is normed up, its rounding too)
+TOL = {"float32": 5e-5, "bfloat16": 0.12}       # of the spread of the oracle's logits, for every row,
+MEDIAN = {"float32": 2e-5, "bfloat16": 0.03}    # and for the middle one (a head whose read-out is nearly nothing is normed up, and its rounding with it)
 
 
 def calm(oracle, seed, n, vocab):
@@ -645,7 +646,7 @@ def calm(oracle, seed, n, vocab):
             before = ([dict(m) for m in oracle.memory], oracle.fed)
             token = int(torch.randint(0, vocab, (1,), generator=gen))
             row = oracle.forward([token])[0]
-            if oracle.margin > 0.08:
+            if oracle.margin > 0.12:
                 break
             oracle.memory, oracle.fed = before
         else:
@@ -680,13 +681,15 @@ def replayer(folder, dtype, max_tokens):
 
 
 def check(got, oracle_rows, dtype):
-    """Every row's root mean square difference within `TOL` of the logits' spread."""
+    """Every row's root mean square difference within `TOL` of the logits' spread, and the middle row's within `MEDIAN`."""
     assert got, "nothing was compared"
     spread = float(torch.cat([o.flatten() for o in oracle_rows]).std())
     errors = {key: float((row.double().cpu() - oracle_rows[key[0]][key[1]]).pow(2).mean().sqrt()) / spread for key, row in got.items()}
     over = {key: e for key, e in errors.items() if not e <= TOL[dtype]}
     print(f"[{dtype}] worst row {max(errors.values()):.3e} of the logits' spread ({spread:.2f}) over {len(got)} rows")
     assert not over, f"(request, position): error {over}"
+    middle = sorted(errors.values())[(len(errors) - 1) // 2]
+    assert middle <= MEDIAN[dtype], f"half the rows are {middle:.3e} away or more"
 
 
 @pytest.mark.parametrize("dtype", ["float32", "bfloat16"])

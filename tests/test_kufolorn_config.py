@@ -115,7 +115,7 @@ def test_checkpoint_names_and_shapes(tmp_path):
     assert torch.equal(conv[:, 32:60], tensors["l0.mix.v.conv"][28:56].t().float()) and float(conv[:, 60:64].abs().max()) == 0.0
     assert torch.equal(conv[:, 160:180], tensors["l0.mix.k.conv"][20:40].t().float()) and torch.equal(conv[:, 192:212], tensors["l0.mix.q.conv"][:20].t().float())
     # the head reads the embedding's table, capped
-    assert model.head.weight is model.embedding.weight and model.head.softcap == 9.0
+    assert model.head.weight is model.embedding.weight and model.head.softcap == 2.0
 
 
 def test_parts_refuse_what_they_cannot_do():

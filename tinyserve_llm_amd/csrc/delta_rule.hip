@@ -326,6 +326,7 @@ extern "C" int ts_delta_step(float* out, const void* mixed, int dtype, const flo
 // ---- chunks of 64 tokens on the matrix cores (bfloat16) ----------------------------------------------------------
 
 #define DL_TILE (SS_L * SS_L)   // a chunk's T or its weights, one bfloat16 term of them
+#define DL_SCALES 5             // numbers of a chunk's token beside its rows
 #define DL_F 68                 // a row of 64 numbers in shared memory, 32-bit
 
 // D += A B over 4 k, 32-bit: lane (r, q) gives A[r][q] and B[q][r]; it gets D[4 q + i][r].
@@ -351,19 +352,24 @@ static __device__ __forceinline__ void dl_put(float* dst, const float4_t& m, flo
   for (int i = 0; i < 4; ++i) dst[(4 * q + i) * DL_F + r] = sign * m[i];
 }
 
+// What the walk reads lies in pieces: 16 rows by 32 of an operand as a wave takes them, lane after lane eight numbers of
+// 2 bytes (lane (r, q): row r, columns 8 q .. 8 q + 7), a kilobyte side by side.
+#define DL_PIECE (TS_WAVE * 8)
+
 // One workgroup per (chunk, head). chunks: int32 [chunks, 4] (first token of the step, tokens 1 .. 64, request, whether the
-// request's last). Per chunk and head: inv [2][64][64] (T in two terms, rows tokens), wts [2][64][64] (the second sum's
-// weights in two terms), vt [vp][64] (v turned), scales [4][64] (beta, beta exp(b) / |k|, exp(b) / |q| dim^(-1/2),
-// exp(b_L - b) / |k|; zeros for tokens past the chunk's end), totals (exp(b_L)); per chunk and group: kt [np][64] (k turned).
+// request's last). Per chunk and head: inv (T, rows tokens, as pieces [16 tokens][term][32 columns]), wts (the second sum's
+// weights likewise; of both the pieces above the diagonal are never written nor read), vt (v, [16 value columns][16 tokens]
+// [lane][4 tokens]), scales [5][64] (beta, beta exp(b) / |k|, exp(b) / |q| dim^(-1/2), exp(b_L - b) / |k|, zeros for tokens
+// past the chunk's end; exp(b_L), 64 times); per chunk and group: keys (k and q as pieces [16 tokens][32 places], then k
+// turned round as pieces [16 places][32 tokens]).
 template <int NQ>
-__global__ void __launch_bounds__(DL_THREADS)
-delta_chunk_solve_kernel(bf16_t* __restrict__ inv, bf16_t* __restrict__ wts, bf16_t* __restrict__ kt, bf16_t* __restrict__ vt,
-                         float* __restrict__ scales, float* __restrict__ totals, const bf16_t* __restrict__ mixed,
-                         const float* __restrict__ units, const float* __restrict__ betas, const float* __restrict__ logs,
+__global__ void __launch_bounds__(DL_THREADS, 4)
+delta_chunk_solve_kernel(bf16_t* __restrict__ inv, bf16_t* __restrict__ wts, bf16_t* __restrict__ keys, bf16_t* __restrict__ vt,
+                         float* __restrict__ scales, const bf16_t* __restrict__ mixed, const float* __restrict__ units, const float* __restrict__ betas, const float* __restrict__ logs,
                          const int32_t* __restrict__ chunks, int heads, int vp, int groups) {
   constexpr int np = 32 * NQ;
   __shared__ __attribute__((aligned(16))) float a_s[SS_L][DL_F], t_s[SS_L][DL_F];
-  __shared__ __attribute__((aligned(16))) bf16_t turn_s[64][SS_PAD];
+  bf16_t (*turn_s)[SS_PAD] = (bf16_t (*)[SS_PAD])a_s;          // (at the end, where a_s has been read)
   __shared__ double b_s[SS_L];
   __shared__ float rk_s[SS_L], rq_s[SS_L], beta_s[SS_L];
   const int chunk = blockIdx.x, h = blockIdx.y;
@@ -373,6 +379,7 @@ delta_chunk_solve_kernel(bf16_t* __restrict__ inv, bf16_t* __restrict__ wts, bf1
   const int64_t ch = (int64_t)chunk * heads + h;
   const bf16_t* k_rows = mixed + (int64_t)tok0 * row + heads * vp + g * np + 8 * q;
   const bf16_t* q_rows = k_rows + groups * np;
+  bf16_t* own_keys = keys + ((int64_t)chunk * groups + g) * 3 * np * SS_L;
   const int t = 16 * wave + r;                               // (this lane's token of the products)
   const int tc = min(t, len - 1);
   if (threadIdx.x < TS_WAVE) {
@@ -386,12 +393,12 @@ delta_chunk_solve_kernel(bf16_t* __restrict__ inv, bf16_t* __restrict__ wts, bf1
     rk_s[lane] = rk;
     rq_s[lane] = rq;
     beta_s[lane] = beta;
-    float* sc = scales + ch * 4 * SS_L + lane;
+    float* sc = scales + ch * DL_SCALES * SS_L + lane;
     sc[0] = there ? beta : 0.f;
     sc[SS_L] = there ? beta * grown * rk : 0.f;
     sc[2 * SS_L] = there ? grown * rq : 0.f;
     sc[3 * SS_L] = there ? expf((float)(last - b)) * rk : 0.f;
-    if (lane == 0) totals[ch] = expf((float)last);
+    sc[4 * SS_L] = expf((float)last);
   }
   // k_j . k_t and k_j . q_t, keys as the products' rows: lane (r, q) gets keys 16 jb + 4 q .. + 3 of token t
   float4_t kk[4], kq[4];
@@ -401,6 +408,14 @@ delta_chunk_solve_kernel(bf16_t* __restrict__ inv, bf16_t* __restrict__ wts, bf1
     for (int i = 0; i < NQ; ++i) {
       kf[i] = *(const uint4*)(k_rows + (int64_t)tc * row + 32 * i);
       qf[i] = *(const uint4*)(q_rows + (int64_t)tc * row + 32 * i);
+    }
+    if (h == g * per) {                                      // (the first head of a group leaves the group's pieces)
+      bf16_t* piece = own_keys + (wave * NQ) * DL_PIECE + lane * 8;
+#pragma unroll
+      for (int i = 0; i < NQ; ++i) {
+        *(uint4*)(piece + i * DL_PIECE) = kf[i];
+        *(uint4*)(piece + i * DL_PIECE + np * SS_L) = qf[i];
+      }
     }
 #pragma unroll
     for (int jb = 0; jb < 4; ++jb) {
@@ -419,7 +434,8 @@ delta_chunk_solve_kernel(bf16_t* __restrict__ inv, bf16_t* __restrict__ wts, bf1
   {
     const double bt = b_s[t];
     const float kscale = beta_s[t] * rk_s[t], qscale = rq_s[t];
-    bf16_t* w_row = wts + ch * 2 * DL_TILE + t * SS_L + 4 * q;
+    // keys 16 jb + 4 q .. + 3 of a token are half of what lane (r, 2 (jb & 1) + q / 2) of piece jb / 2 holds
+    bf16_t* w_piece = wts + ch * 2 * DL_TILE + wave * 4 * DL_PIECE + ((q >> 1) * 16 + r) * 8 + 4 * (q & 1);
 #pragma unroll
     for (int jb = 0; jb < 4; ++jb) {
       float a[4], p[4];
@@ -432,13 +448,11 @@ delta_chunk_solve_kernel(bf16_t* __restrict__ inv, bf16_t* __restrict__ wts, bf1
         p[i] = upto ? qscale * fade * kq[jb][i] : 0.f;
       }
       ss_store4(&a_s[t][16 * jb + 4 * q], a);
-      if (jb <= wave) {
+      if (jb <= (wave | 1)) {                                // (beyond the diagonal's piece: nobody reads)
+        bf16_t* dst = w_piece + (jb >> 1) * DL_PIECE + (jb & 1) * 32 * 8;
         const uint32_t h0 = pack_bf16(p[0], p[1]), h1 = pack_bf16(p[2], p[3]);
-        *(uint2*)(w_row + 16 * jb) = make_uint2(h0, h1);
-        *(uint2*)(w_row + DL_TILE + 16 * jb) = make_uint2(ss_rest(h0, p[0], p[1]), ss_rest(h1, p[2], p[3]));
-      } else {                                               // (above the diagonal: zeros)
-        *(uint2*)(w_row + 16 * jb) = make_uint2(0, 0);
-        *(uint2*)(w_row + DL_TILE + 16 * jb) = make_uint2(0, 0);
+        *(uint2*)dst = make_uint2(h0, h1);
+        *(uint2*)(dst + 2 * DL_PIECE) = make_uint2(ss_rest(h0, p[0], p[1]), ss_rest(h1, p[2], p[3]));
       }
     }
   }
@@ -480,30 +494,50 @@ delta_chunk_solve_kernel(bf16_t* __restrict__ inv, bf16_t* __restrict__ wts, bf1
   }
   __syncthreads();
   {
-    bf16_t* t_row = inv + ch * 2 * DL_TILE;
-    for (int at = threadIdx.x; at < DL_TILE / 4; at += DL_THREADS) {
-      const int i = at >> 4, j = 4 * (at & 15);
-      float x[4] = {0.f, 0.f, 0.f, 0.f};
-      if ((j >> 4) <= (i >> 4)) ss_load4(&t_s[i][j], x);     // (the blocks above the diagonal were never written)
-      const uint32_t h0 = pack_bf16(x[0], x[1]), h1 = pack_bf16(x[2], x[3]);
-      *(uint2*)(t_row + i * SS_L + j) = make_uint2(h0, h1);
-      *(uint2*)(t_row + DL_TILE + i * SS_L + j) = make_uint2(ss_rest(h0, x[0], x[1]), ss_rest(h1, x[2], x[3]));
+    bf16_t* t_piece = inv + ch * 2 * DL_TILE + wave * 4 * DL_PIECE + lane * 8;
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk) {
+      if (kk == 1 && wave < 2) continue;
+      float x[2][4];
+#pragma unroll
+      for (int half = 0; half < 2; ++half) {
+        const int j = 32 * kk + 8 * q + 4 * half;
+        if ((j >> 4) <= wave) ss_load4(&t_s[t][j], x[half]); // (the blocks above the diagonal were never written)
+        else x[half][0] = x[half][1] = x[half][2] = x[half][3] = 0.f;
+      }
+      uint4 hi, lo;
+#pragma unroll
+      for (int k = 0; k < 4; ++k) {
+        const float a = x[k >> 1][2 * (k & 1)], b = x[k >> 1][2 * (k & 1) + 1];
+        (&hi.x)[k] = pack_bf16(a, b);
+        (&lo.x)[k] = ss_rest((&hi.x)[k], a, b);
+      }
+      *(uint4*)(t_piece + kk * DL_PIECE) = hi;
+      *(uint4*)(t_piece + (2 + kk) * DL_PIECE) = lo;
     }
   }
-  // v and (by the first head of a group) k turned round
-  auto turn = [&](bf16_t* dst, const bf16_t* src, int cols) {
+  // v and (by the first head of a group) k turned round, 64 columns at a time
+  auto turn = [&](const bf16_t* src, int cols, auto leave) {
     for (int c0 = 0; c0 < cols; c0 += 64) {
       __syncthreads();                                       // (the tile before has been read)
       ss_turn<false>(turn_s, nullptr, src + c0, row, tok0, len, cols - c0, nullptr);
       __syncthreads();
-      for (int at = threadIdx.x; at < 64 * SS_L / 8; at += DL_THREADS) {
-        const int c = at >> 3, piece = 8 * (at & 7);
-        if (c0 + c < cols) *(uint4*)(dst + (int64_t)(c0 + c) * SS_L + piece) = *(const uint4*)&turn_s[c][piece];
-      }
+      leave(c0);
     }
   };
-  turn(vt + ch * vp * SS_L, mixed + h * vp, vp);
-  if (h == g * per) turn(kt + ((int64_t)chunk * groups + g) * np * SS_L, mixed + heads * vp + g * np, np);
+  bf16_t* own_v = vt + ch * vp * SS_L;
+  turn(mixed + h * vp, vp, [&](int c0) {
+#pragma unroll
+    for (int c = 0; c < 4; ++c)                              // (wave w: tokens 16 w .. + 15 of the tile's columns, 16 at a time)
+      if (c0 + 16 * c < vp) *(uint2*)(own_v + ((c0 / 16 + c) * 4 + wave) * TS_WAVE * 4 + lane * 4) = *(const uint2*)&turn_s[16 * c + r][16 * wave + 4 * q];
+  });
+  if (h == g * per)
+    turn(mixed + heads * vp + g * np, np, [&](int c0) {
+      if (c0 + 16 * wave >= np) return;
+#pragma unroll
+      for (int kk = 0; kk < 2; ++kk)
+        *(uint4*)(own_keys + 2 * np * SS_L + ((c0 / 16 + wave) * 2 + kk) * DL_PIECE + lane * 8) = *(const uint4*)&turn_s[16 * wave + r][32 * kk + 8 * q];
+    });
 }
 
 // A number's two bfloat16 terms, four at a time.
@@ -516,32 +550,39 @@ static __device__ __forceinline__ void dl_split4(bf16_t* hi, bf16_t* lo, const f
 // One workgroup per (request and head, 16 value columns); it walks the request's chunks in order. Wave w has the chunk's
 // tokens 16 w .. 16 w + 15 and of the state the blocks of 16 key places w, w + 4, ... (32-bit, in registers); what the next
 // product needs whole goes through shared memory in two terms, laid out as that product's operand. The next chunk's
-// operands are fetched while one is worked on.
+// operands are fetched while one is worked on. Between two barriers everything that lies in shared memory is asked for
+// before the first of it is used, and a product's terms go into sums of their own, so that no product waits for another.
 template <int NQ>
-__global__ void __launch_bounds__(DL_THREADS)
+__global__ void __launch_bounds__(DL_THREADS, NQ <= 4 ? 2 : 1)
 delta_chunk_walk_kernel(float* __restrict__ out, const bf16_t* __restrict__ inv, const bf16_t* __restrict__ wts,
-                        const bf16_t* __restrict__ kt, const bf16_t* __restrict__ vt, const float* __restrict__ scales,
-                        const float* __restrict__ totals, const bf16_t* __restrict__ mixed, float* __restrict__ states,
-                        int64_t slot_stride, const int32_t* __restrict__ chunks, const int32_t* __restrict__ chunk_cu,
-                        const int32_t* __restrict__ state_slots, int heads, int vdim, int vp, int groups) {
+                        const bf16_t* __restrict__ keys, const bf16_t* __restrict__ vt, const float* __restrict__ scales,
+                        float* __restrict__ states, int64_t slot_stride, const int32_t* __restrict__ chunks,
+                        const int32_t* __restrict__ chunk_cu, const int32_t* __restrict__ state_slots, int num_seqs, int heads, int vdim,
+                        int vp, int groups) {
   constexpr int np = 32 * NQ, BLOCKS = (2 * NQ + 3) / 4, S_ROW = np + 8;
   __shared__ __attribute__((aligned(16))) bf16_t s_s[2][16][S_ROW];            // the state: [term][column][place]
   __shared__ __attribute__((aligned(16))) bf16_t r_s[2][16][SS_PAD];           // beta V - beta exp(b) K S0: [term][column][token]
   __shared__ __attribute__((aligned(16))) bf16_t u_s[2][16][SS_PAD], d_s[2][16][SS_PAD];     // U, and U fading to the chunk's end
-  const int seq = blockIdx.x / heads, h = blockIdx.x - seq * heads, v0 = 16 * blockIdx.y;
+  // the slices of one head run on one die (workgroup index mod 8), side by side, and share what they read in its cache
+  const int slices = vp / 16, die = blockIdx.x % 8, turn = blockIdx.x / 8;
+  const int pair = (turn / slices) * 8 + die, slice = turn % slices;
+  if (pair >= num_seqs * heads) return;
+  const int seq = pair / heads, h = pair - seq * heads, v0 = 16 * slice;
   const int begin = chunk_cu[seq], end = chunk_cu[seq + 1];
   if (begin >= end) return;
-  const int row = heads * vp + 2 * groups * np, g = h / (heads / groups);
+  const int g = h / (heads / groups);
   const int wave = wave_index(), lane = threadIdx.x & (TS_WAVE - 1), r = lane & 15, q = lane >> 4;
   float* st = states + (int64_t)state_slots[seq] * slot_stride + (int64_t)h * vp * np + (int64_t)(v0 + r) * np + 4 * q;
-  float S[BLOCKS][4];
+  const float4_t none = {0.f, 0.f, 0.f, 0.f};
+  auto has = [&](int i) { return (2 * NQ) % 4 == 0 || wave + 4 * i < 2 * NQ; };              // whether this wave has an i-th block
+  float4_t S[BLOCKS];
 #pragma unroll
   for (int i = 0; i < BLOCKS; ++i) {
-    const int blk = wave + 4 * i;
-    S[i][0] = S[i][1] = S[i][2] = S[i][3] = 0.f;
-    if (blk < 2 * NQ) {
-      ss_load4(st + 16 * blk, S[i]);
-      dl_split4(&s_s[0][r][16 * blk + 4 * q], &s_s[1][r][16 * blk + 4 * q], S[i]);
+    S[i] = none;
+    if (has(i)) {
+      S[i] = *(const float4_t*)(st + 16 * (wave + 4 * i));
+      const float x[4] = {S[i][0], S[i][1], S[i][2], S[i][3]};
+      dl_split4(&s_s[0][r][16 * (wave + 4 * i) + 4 * q], &s_s[1][r][16 * (wave + 4 * i) + 4 * q], x);
     }
   }
   const bool second = wave >= 2;                             // whether this wave's tokens see the chunk's second half
@@ -549,140 +590,178 @@ delta_chunk_walk_kernel(float* __restrict__ out, const bf16_t* __restrict__ inv,
     uint4 k[NQ], qq[NQ], t[2][2], w[2][2], kt[BLOCKS][2];
     uint2 v;
     float beta[4], bk[4], bq[4], dk[4], total;
-    int tok0, len;
   };
+  // (a request's chunks lie side by side, all of 64 tokens but the last)
+  const int first = chunks[4 * begin], stop = chunks[4 * end - 4] + chunks[4 * end - 3];
   auto fetch = [&](int c, Operands& o) {
-    o.tok0 = chunks[4 * c];
-    o.len = chunks[4 * c + 1];
     const int64_t ch = (int64_t)c * heads + h;
-    const bf16_t* k_row = mixed + (int64_t)(o.tok0 + min(16 * wave + r, o.len - 1)) * row + heads * vp + g * np + 8 * q;
-    const bf16_t* t_row = inv + ch * 2 * DL_TILE + (16 * wave + r) * SS_L + 8 * q;
-    const bf16_t* w_row = wts + ch * 2 * DL_TILE + (16 * wave + r) * SS_L + 8 * q;
+    const bf16_t* k_piece = keys + ((int64_t)c * groups + g) * 3 * np * SS_L + lane * 8;
+    const bf16_t* t_piece = inv + ch * 2 * DL_TILE + wave * 4 * DL_PIECE + lane * 8;
+    const bf16_t* w_piece = wts + ch * 2 * DL_TILE + wave * 4 * DL_PIECE + lane * 8;
 #pragma unroll
     for (int i = 0; i < NQ; ++i) {
-      o.k[i] = *(const uint4*)(k_row + 32 * i);
-      o.qq[i] = *(const uint4*)(k_row + groups * np + 32 * i);
+      o.k[i] = *(const uint4*)(k_piece + (wave * NQ + i) * DL_PIECE);
+      o.qq[i] = *(const uint4*)(k_piece + np * SS_L + (wave * NQ + i) * DL_PIECE);
     }
 #pragma unroll
-    for (int term = 0; term < 2; ++term)
+    for (int kk = 0; kk < 2; ++kk) {
+      if (kk == 1 && !second) continue;
 #pragma unroll
-      for (int kk = 0; kk < 2; ++kk) {
-        o.t[term][kk] = *(const uint4*)(t_row + term * DL_TILE + 32 * kk);
-        o.w[term][kk] = *(const uint4*)(w_row + term * DL_TILE + 32 * kk);
+      for (int term = 0; term < 2; ++term) {
+        o.t[term][kk] = *(const uint4*)(t_piece + (2 * term + kk) * DL_PIECE);
+        o.w[term][kk] = *(const uint4*)(w_piece + (2 * term + kk) * DL_PIECE);
       }
-    o.v = *(const uint2*)(vt + (ch * vp + v0 + r) * SS_L + 16 * wave + 4 * q);
-    const float* sc = scales + ch * 4 * SS_L + 16 * wave + 4 * q;
+    }
+    o.v = *(const uint2*)(vt + ch * vp * SS_L + (slice * 4 + wave) * TS_WAVE * 4 + lane * 4);
+    const float* sc = scales + ch * DL_SCALES * SS_L + 16 * wave + 4 * q;
     ss_load4(sc, o.beta);
     ss_load4(sc + SS_L, o.bk);
     ss_load4(sc + 2 * SS_L, o.bq);
     ss_load4(sc + 3 * SS_L, o.dk);
-    o.total = totals[ch];
+    o.total = sc[4 * SS_L];
 #pragma unroll
     for (int i = 0; i < BLOCKS; ++i) {
-      const int blk = min(wave + 4 * i, 2 * NQ - 1);
-      const bf16_t* kt_row = kt + (((int64_t)c * groups + g) * np + 16 * blk + r) * SS_L + 8 * q;
+      const bf16_t* turned = k_piece + 2 * np * SS_L + min(wave + 4 * i, 2 * NQ - 1) * 2 * DL_PIECE;
 #pragma unroll
-      for (int kk = 0; kk < 2; ++kk) o.kt[i][kk] = *(const uint4*)(kt_row + 32 * kk);
+      for (int kk = 0; kk < 2; ++kk) o.kt[i][kk] = *(const uint4*)(turned + kk * DL_PIECE);
     }
   };
-  Operands now, next;
-  fetch(begin, now);
-  for (int c = begin; c < end; ++c) {
-    fetch(min(c + 1, end - 1), next);
+  auto work = [&](int c, const Operands& now) {
     __syncthreads();                                         // (the state lies in s_s)
-    float4_t x = {0.f, 0.f, 0.f, 0.f}, y = {0.f, 0.f, 0.f, 0.f};
+    float4_t x[2] = {none, none}, y[2] = {none, none};
+    constexpr int AT_ONCE = NQ == 4 ? 2 : 4;                               // pieces of the state whose two terms are read together
 #pragma unroll
-    for (int i = 0; i < NQ; ++i)
+    for (int i0 = 0; i0 < NQ; i0 += AT_ONCE) {
+      uint4 s[AT_ONCE][2];
 #pragma unroll
-      for (int term = 0; term < 2; ++term) {
-        const uint4 s = *(const uint4*)&s_s[term][r][32 * i + 8 * q];
-        x = mfma32(now.k[i], s, x);
-        y = mfma32(now.qq[i], s, y);
-      }
+      for (int i = 0; i < AT_ONCE && i0 + i < NQ; ++i)
+#pragma unroll
+        for (int term = 0; term < 2; ++term) s[i][term] = *(const uint4*)&s_s[term][r][32 * (i0 + i) + 8 * q];
+#pragma unroll
+      for (int i = 0; i < AT_ONCE && i0 + i < NQ; ++i)
+#pragma unroll
+        for (int term = 0; term < 2; ++term) {
+          x[term] = mfma32(now.k[i0 + i], s[i][term], x[term]);
+          y[term] = mfma32(now.qq[i0 + i], s[i][term], y[term]);
+        }
+    }
     {
       const float v[4] = {__uint_as_float(now.v.x << 16), __uint_as_float(now.v.x & 0xffff0000u), __uint_as_float(now.v.y << 16),
                           __uint_as_float(now.v.y & 0xffff0000u)};
       float rest[4];
 #pragma unroll
-      for (int i = 0; i < 4; ++i) {
-        rest[i] = fmaf(now.beta[i], v[i], -now.bk[i] * x[i]);
-        y[i] *= now.bq[i];
-      }
+      for (int i = 0; i < 4; ++i) rest[i] = fmaf(now.beta[i], v[i], -now.bk[i] * (x[0][i] + x[1][i]));
       dl_split4(&r_s[0][r][16 * wave + 4 * q], &r_s[1][r][16 * wave + 4 * q], rest);
     }
     __syncthreads();
-    float4_t u = {0.f, 0.f, 0.f, 0.f};
+    // rows of T and of the weights beyond this wave's tokens are zeros: the second half counts for waves 2 and 3 alone
+    uint4 rest[2][2];
 #pragma unroll
-    for (int kk = 0; kk < 2; ++kk) {
-      if (kk == 1 && !second) continue;
-      const uint4 hi = *(const uint4*)&r_s[0][r][32 * kk + 8 * q], lo = *(const uint4*)&r_s[1][r][32 * kk + 8 * q];
-      u = mfma32(now.t[0][kk], hi, u);
-      u = mfma32(now.t[0][kk], lo, u);
-      u = mfma32(now.t[1][kk], hi, u);
+    for (int kk = 0; kk < 2; ++kk)
+#pragma unroll
+      for (int term = 0; term < 2; ++term) rest[kk][term] = *(const uint4*)&r_s[term][r][32 * kk + 8 * q];
+    float4_t u0 = mfma32(now.t[0][0], rest[0][0], none), u1 = mfma32(now.t[0][0], rest[0][1], none), u2 = mfma32(now.t[1][0], rest[0][0], none);
+    if (second) {
+      u0 = mfma32(now.t[0][1], rest[1][0], u0);
+      u1 = mfma32(now.t[0][1], rest[1][1], u1);
+      u2 = mfma32(now.t[1][1], rest[1][0], u2);
     }
     {
-      const float w[4] = {u[0], u[1], u[2], u[3]}, fading[4] = {u[0] * now.dk[0], u[1] * now.dk[1], u[2] * now.dk[2], u[3] * now.dk[3]};
-      dl_split4(&u_s[0][r][16 * wave + 4 * q], &u_s[1][r][16 * wave + 4 * q], w);
-      dl_split4(&d_s[0][r][16 * wave + 4 * q], &d_s[1][r][16 * wave + 4 * q], fading);
-    }
-    __syncthreads();
-#pragma unroll
-    for (int i = 0; i < BLOCKS; ++i) {
-      const int blk = wave + 4 * i;
-      if (blk >= 2 * NQ) continue;
-      float4_t s = {now.total * S[i][0], now.total * S[i][1], now.total * S[i][2], now.total * S[i][3]};
-#pragma unroll
-      for (int kk = 0; kk < 2; ++kk)
-#pragma unroll
-        for (int term = 0; term < 2; ++term) s = mfma32(now.kt[i][kk], *(const uint4*)&d_s[term][r][32 * kk + 8 * q], s);
-#pragma unroll
-      for (int j = 0; j < 4; ++j) S[i][j] = s[j];
-      dl_split4(&s_s[0][r][16 * blk + 4 * q], &s_s[1][r][16 * blk + 4 * q], S[i]);
-    }
-#pragma unroll
-    for (int kk = 0; kk < 2; ++kk) {
-      if (kk == 1 && !second) continue;
-      const uint4 hi = *(const uint4*)&u_s[0][r][32 * kk + 8 * q], lo = *(const uint4*)&u_s[1][r][32 * kk + 8 * q];
-      y = mfma32(now.w[0][kk], hi, y);
-      y = mfma32(now.w[0][kk], lo, y);
-      y = mfma32(now.w[1][kk], hi, y);
-    }
-    if (v0 + r < vdim) {
+      float w[4], fading[4];
 #pragma unroll
       for (int i = 0; i < 4; ++i) {
-        const int tok = 16 * wave + 4 * q + i;
-        if (tok < now.len) out[((int64_t)(now.tok0 + tok) * heads + h) * vdim + v0 + r] = y[i];
+        w[i] = u0[i] + (u1[i] + u2[i]);
+        fading[i] = w[i] * now.dk[i];
       }
+      dl_split4(&d_s[0][r][16 * wave + 4 * q], &d_s[1][r][16 * wave + 4 * q], fading);
+      dl_split4(&u_s[0][r][16 * wave + 4 * q], &u_s[1][r][16 * wave + 4 * q], w);
     }
-    now = next;
+#pragma unroll
+    for (int i = 0; i < 4; ++i) {                            // (while the other waves come to the barrier)
+      y[0][i] = now.bq[i] * (y[0][i] + y[1][i]);
+#pragma unroll
+      for (int b = 0; b < BLOCKS; ++b) S[b][i] *= now.total;
+    }
+    __syncthreads();
+    uint4 d[2][2], w[2][2];
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk)
+#pragma unroll
+      for (int term = 0; term < 2; ++term) d[kk][term] = *(const uint4*)&d_s[term][r][32 * kk + 8 * q];
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk)
+#pragma unroll
+      for (int term = 0; term < 2; ++term) w[kk][term] = *(const uint4*)&u_s[term][r][32 * kk + 8 * q];
+    float4_t low[BLOCKS];
+#pragma unroll
+    for (int i = 0; i < BLOCKS; ++i) low[i] = none;
+#pragma unroll
+    for (int kk = 0; kk < 2; ++kk)
+#pragma unroll
+      for (int i = 0; i < BLOCKS; ++i) {
+        S[i] = mfma32(now.kt[i][kk], d[kk][0], S[i]);
+        low[i] = mfma32(now.kt[i][kk], d[kk][1], low[i]);
+      }
+    y[0] = mfma32(now.w[0][0], w[0][0], y[0]);
+    y[1] = mfma32(now.w[0][0], w[0][1], none);
+    float4_t y2 = mfma32(now.w[1][0], w[0][0], none);
+    if (second) {
+      y[0] = mfma32(now.w[0][1], w[1][0], y[0]);
+      y[1] = mfma32(now.w[0][1], w[1][1], y[1]);
+      y2 = mfma32(now.w[1][1], w[1][0], y2);
+    }
+#pragma unroll
+    for (int i = 0; i < BLOCKS; ++i) {
+#pragma unroll
+      for (int j = 0; j < 4; ++j) S[i][j] += low[i][j];
+      const float x4[4] = {S[i][0], S[i][1], S[i][2], S[i][3]};
+      if (has(i)) dl_split4(&s_s[0][r][16 * (wave + 4 * i) + 4 * q], &s_s[1][r][16 * (wave + 4 * i) + 4 * q], x4);
+    }
+    if (v0 + r < vdim) {
+      const int tok = first + SS_L * (c - begin) + 16 * wave + 4 * q;
+      float* dst = out + ((int64_t)tok * heads + h) * vdim + v0 + r;
+#pragma unroll
+      for (int i = 0; i < 4; ++i)
+        if (tok + i < stop) dst[(int64_t)i * heads * vdim] = y[0][i] + (y[1][i] + y2[i]);
+    }
+  };
+  Operands even, odd;                                        // (two sets in turn: nothing is copied from one to the other)
+  fetch(begin, even);
+  for (int c = begin; c < end; c += 2) {
+    fetch(min(c + 1, end - 1), odd);
+    work(c, even);
+    if (c + 1 >= end) break;
+    fetch(min(c + 2, end - 1), even);
+    work(c + 1, odd);
   }
 #pragma unroll
-  for (int i = 0; i < BLOCKS; ++i) {
-    const int blk = wave + 4 * i;
-    if (blk < 2 * NQ) ss_store4(st + 16 * blk, S[i]);
-  }
+  for (int i = 0; i < BLOCKS; ++i)
+    if (has(i)) *(float4_t*)(st + 16 * (wave + 4 * i)) = S[i];
 }
 
 // chunk_cu: int32 [requests + 1], each request's first chunk; requests without chunks keep their state as it is. inv and wts
-// bfloat16 [chunks, heads, 2, 64, 64], kt [chunks, groups, np, 64], vt [chunks, heads, vp, 64], scales float32 [chunks, heads,
-// 4, 64], totals [chunks, heads]: scratch.
+// bfloat16 [chunks, heads, 2, 64, 64], keys [chunks, groups, 3, np, 64], vt [chunks, heads, vp, 64], scales float32 [chunks, heads,
+// 5, 64]: scratch.
 extern "C" int ts_delta_chunks(float* out, const void* mixed, const float* units, const float* betas, const float* logs, float* states,
                                int64_t slot_stride, const int32_t* chunks, const int32_t* chunk_cu, const int32_t* state_slots,
-                               void* inv, void* wts, void* kt, void* vt, float* scales, float* totals, int num_chunks, int num_seqs,
-                               int heads, int vdim, int vp, int groups, int np, hipStream_t stream) {
+                               void* inv, void* wts, void* keys, void* vt, float* scales, int num_chunks, int num_seqs, int heads,
+                               int vdim, int vp, int groups, int np, hipStream_t stream) {
   if (num_chunks <= 0 || num_seqs <= 0) return TS_OK;
   if (heads <= 0 || heads > 65535 || groups <= 0 || heads % groups || vdim <= 0 || vp < vdim || vp % 16 || np <= 0 || np % 32 ||
-      np > DL_MAX_CHUNK_NP || (int64_t)num_seqs * heads > 0x7fffffff || vp / 16 > 65535 || slot_stride < (int64_t)heads * vp * np || slot_stride % 4 ||
-      (((uintptr_t)states | (uintptr_t)mixed | (uintptr_t)inv | (uintptr_t)wts | (uintptr_t)kt | (uintptr_t)vt | (uintptr_t)scales) & 15))
+      np > DL_MAX_CHUNK_NP || slot_stride < (int64_t)heads * vp * np || slot_stride % 4 ||
+      (((uintptr_t)states | (uintptr_t)mixed | (uintptr_t)inv | (uintptr_t)wts | (uintptr_t)keys | (uintptr_t)vt | (uintptr_t)scales) & 15))
     return TS_BAD_SHAPE;
   const bf16_t* m = (const bf16_t*)mixed;
+  const int64_t walkers64 = ((int64_t)num_seqs * heads + 7) / 8 * 8 * (vp / 16);
+  if (walkers64 > 0x7fffffff) return TS_BAD_SHAPE;
+  const unsigned walkers = (unsigned)walkers64;
 #define DL_CHUNKS(NQ) \
   case NQ: \
-    delta_chunk_solve_kernel<NQ><<<dim3(num_chunks, heads), DL_THREADS, 0, stream>>>((bf16_t*)inv, (bf16_t*)wts, (bf16_t*)kt, (bf16_t*)vt, scales, \
-                                                                                     totals, m, units, betas, logs, chunks, heads, vp, groups); \
-    delta_chunk_walk_kernel<NQ><<<dim3(num_seqs * heads, vp / 16), DL_THREADS, 0, stream>>>( \
-        out, (const bf16_t*)inv, (const bf16_t*)wts, (const bf16_t*)kt, (const bf16_t*)vt, scales, totals, m, states, slot_stride, chunks, \
-        chunk_cu, state_slots, heads, vdim, vp, groups); \
+    delta_chunk_solve_kernel<NQ><<<dim3(num_chunks, heads), DL_THREADS, 0, stream>>>((bf16_t*)inv, (bf16_t*)wts, (bf16_t*)keys, (bf16_t*)vt, scales, \
+                                                                                     m, units, betas, logs, chunks, heads, vp, groups); \
+    delta_chunk_walk_kernel<NQ><<<walkers, DL_THREADS, 0, stream>>>(out, (const bf16_t*)inv, (const bf16_t*)wts, (const bf16_t*)keys, \
+                                                                    (const bf16_t*)vt, scales, states, slot_stride, chunks, chunk_cu, state_slots, \
+                                                                    num_seqs, heads, vdim, vp, groups); \
     break;
   switch (np / 32) { DL_CHUNKS(1) DL_CHUNKS(2) DL_CHUNKS(3) DL_CHUNKS(4) DL_CHUNKS(5) DL_CHUNKS(6) DL_CHUNKS(7) DL_CHUNKS(8) }
 #undef DL_CHUNKS

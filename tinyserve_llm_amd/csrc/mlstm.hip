@@ -177,6 +177,37 @@ mlstm_finish_kernel(TO* __restrict__ out, const float* __restrict__ o, const flo
   }
 }
 
+// The same for heads of up to 256 columns, a multiple of four: LP lanes side by side (a power of two) hold a head, four
+// columns each; everything a lane reads is on its way before the head's sum is taken.
+template <typename TO, int LP>
+__global__ void __launch_bounds__(ML_THREADS)
+mlstm_finish_fours_kernel(TO* __restrict__ out, const float* __restrict__ o, const float* __restrict__ weight,
+                          const float* __restrict__ gate, int64_t gate_stride, int heads, int vdim, float eps, int64_t items,
+                          int weight_head, int silu_gate) {
+  const int64_t gid = (int64_t)blockIdx.x * ML_THREADS + threadIdx.x;
+  const int64_t item = min(gid / LP, items - 1);             // (lanes beyond the last head go along for the sums)
+  const int d = 4 * (int)(gid % LP), dc = min(d, vdim - 4);
+  const int64_t t = item / heads;
+  const int h = (int)(item - t * heads);
+  const float4 x = *(const float4*)(o + item * vdim + dc), g = *(const float4*)(gate + t * gate_stride + h * vdim + dc);
+  float4 w = make_float4(1.f, 1.f, 1.f, 1.f);
+  if (weight) w = *(const float4*)(weight + h * weight_head + dc);
+  float squares = d < vdim ? fmaf(x.x, x.x, fmaf(x.y, x.y, fmaf(x.z, x.z, x.w * x.w))) : 0.f;
+#pragma unroll
+  for (int off = LP / 2; off > 0; off >>= 1) squares += __shfl_xor(squares, off, TS_WAVE);
+  const float inv = 1.0f / sqrtf(squares / (float)vdim + eps);
+  if (gid >= items * LP || d >= vdim) return;
+  auto one = [&](float xv, float gv, float wv) {
+    const float s = 1.0f / (1.0f + expf(-gv));
+    return xv * inv * wv * (silu_gate ? gv * s : s);
+  };
+  const float y[4] = {one(x.x, g.x, w.x), one(x.y, g.y, w.y), one(x.z, g.z, w.z), one(x.w, g.w, w.w)};
+  TO* dst = out + item * vdim + d;
+  if constexpr (sizeof(TO) == 4) *(float4*)dst = make_float4(y[0], y[1], y[2], y[3]);
+  else
+    *(uint2*)dst = make_uint2((uint32_t)f2bf(y[0]) | ((uint32_t)f2bf(y[1]) << 16), (uint32_t)f2bf(y[2]) | ((uint32_t)f2bf(y[3]) << 16));
+}
+
 extern "C" int ts_mlstm_finish(void* out, int out_dtype, const float* o, const float* weight, const float* gate,
                                int64_t gate_stride, int num_tokens, int heads, int vdim, float eps, int weight_head,
                                int silu_gate, hipStream_t stream) {
@@ -185,11 +216,27 @@ extern "C" int ts_mlstm_finish(void* out, int out_dtype, const float* o, const f
   const int64_t items = (int64_t)num_tokens * heads;
   const int64_t blocks = (items + ML_WAVES - 1) / ML_WAVES;
   if (blocks > 0x7fffffff) return TS_BAD_SHAPE;
+  if (out_dtype != 0 && out_dtype != 1) return TS_BAD_DTYPE;
+  if (vdim <= 4 * TS_WAVE && vdim % 4 == 0 && gate_stride % 4 == 0 &&
+      (((uintptr_t)out | (uintptr_t)o | (uintptr_t)gate | (uintptr_t)weight) & 15) == 0 && items * TS_WAVE < (int64_t)0x7fffffff * ML_THREADS) {
+#define ML_FOURS(LP) do { \
+    const unsigned groups = (unsigned)((items * LP + ML_THREADS - 1) / ML_THREADS); \
+    if (out_dtype == 0) \
+      mlstm_finish_fours_kernel<float, LP><<<groups, ML_THREADS, 0, stream>>>((float*)out, o, weight, gate, gate_stride, heads, vdim, eps, items, weight_head, silu_gate); \
+    else \
+      mlstm_finish_fours_kernel<bf16_t, LP><<<groups, ML_THREADS, 0, stream>>>((bf16_t*)out, o, weight, gate, gate_stride, heads, vdim, eps, items, weight_head, silu_gate); \
+  } while (0)
+    if (vdim <= 32) ML_FOURS(8);
+    else if (vdim <= 64) ML_FOURS(16);
+    else if (vdim <= 128) ML_FOURS(32);
+    else ML_FOURS(64);
+#undef ML_FOURS
+    return ts_check_launch();
+  }
   if (out_dtype == 0)
     mlstm_finish_kernel<float><<<(unsigned)blocks, ML_THREADS, 0, stream>>>((float*)out, o, weight, gate, gate_stride, heads, vdim, eps, items, weight_head, silu_gate);
-  else if (out_dtype == 1)
+  else
     mlstm_finish_kernel<bf16_t><<<(unsigned)blocks, ML_THREADS, 0, stream>>>((bf16_t*)out, o, weight, gate, gate_stride, heads, vdim, eps, items, weight_head, silu_gate);
-  else return TS_BAD_DTYPE;
   return ts_check_launch();
 }
 

@@ -93,7 +93,7 @@ def kufolorn_spec(config: KufolornConfig) -> ModelSpec:
                 for j in range(e.experts):
                     _unit_names(ckpt, f"{src}.mlp.e{j}", f"{dst}.ff.", e.ff, index=(j,))
         layers.append(LayerSpec(mixer, ff, norms, "post_norm_stream"))
-    table = PartSpec("table", dict(vocab_size=c.vocab, hidden_size=c.width, float32_stream=True, init=(0.0, 1.0)))
+    table = PartSpec("table", dict(vocab_size=c.vocab, hidden_size=c.width, float32_stream=True, init=(0.0, 0.3)))
     head = PartSpec("projection", dict(vocab_size=c.vocab, hidden_size=c.width, tied=True, softcap=c.logit_softcap))
     return ModelSpec(
         architecture=c.architecture, vocab_size=c.vocab, hidden_size=c.width, max_position=None, layers=layers,

@@ -114,7 +114,7 @@ def _declare(lib: ctypes.CDLL) -> None:
         "ts_retention_prepare": [p, i, p, i64, p, p, i, i, i, i, i, i, i, p],
         "ts_delta_prepare": [p, i, p, p, p, p, i64, p, p, i64, p, p, p, p, p, i, i, i, i, i, i, i, i, f, i, p],
         "ts_delta_step": [p, p, i, p, p, p, p, i64, p, p, i, i, i, i, i, i, i, p],
-        "ts_delta_chunks": [p, p, p, p, p, p, i64, p, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, p],
+        "ts_delta_chunks": [p, p, p, p, p, p, i64, p, p, p, p, p, p, p, p, i, i, i, i, i, i, i, p],
         "ts_soft_cap": [p, f, i64, p],
         "ts_gated_group_norm": [p, i, p, p, i64, p, i, i, i, f, p],
         "ts_mlstm_scan": [p, p, i64, p, p, p, p, p, i, i, i, i, i, f, f, p],
@@ -2864,12 +2864,12 @@ def delta_scan(rows: DeltaRows, state: torch.Tensor, ctx, sizes: SsdSizes, chunk
         chunks, chunk_cu = _step_chunks(ctx, chunks_from, dev)
         C, L = chunks.shape[0], SSD_CHUNK
         tiles = torch.empty((2, C, z.heads, 2, L, L), dtype=torch.bfloat16, device=dev)
-        turned = torch.empty((C, z.groups * z.np + z.heads * z.vp, L), dtype=torch.bfloat16, device=dev)
-        scales = torch.empty((C * z.heads * (4 * L + 1),), dtype=torch.float32, device=dev)
+        rows_again = torch.empty((C, 3 * z.groups * z.np + z.heads * z.vp, L), dtype=torch.bfloat16, device=dev)
+        scales = torch.empty((C, z.heads, 5, L), dtype=torch.float32, device=dev)
         _run("delta_chunks", library().ts_delta_chunks(
             _ptr(out), _ptr(mixed), _ptr(rows.units), _ptr(rows.betas), _ptr(rows.logs), _ptr(state), state.stride(0), _ptr(chunks), _ptr(chunk_cu),
-            _ptr(ctx.state_slots), _ptr(tiles), tiles[1].data_ptr(), _ptr(turned), turned.data_ptr() + 2 * L * C * z.groups * z.np, _ptr(scales),
-            scales.data_ptr() + 4 * 4 * L * C * z.heads, C, S, z.heads, z.vdim, z.vp, z.groups, z.np, _stream()))
+            _ptr(ctx.state_slots), _ptr(tiles), tiles[1].data_ptr(), _ptr(rows_again), rows_again.data_ptr() + 2 * L * C * 3 * z.groups * z.np,
+            _ptr(scales), C, S, z.heads, z.vdim, z.vp, z.groups, z.np, _stream()))
         if _all_in_chunks(ctx, chunks_from):
             return out
     _run("delta_step", library().ts_delta_step(

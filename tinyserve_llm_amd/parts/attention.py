@@ -210,7 +210,7 @@ class GeneralAttention(Mixer):
         specs = {"qkv": ParamSpec((self.projected, self.hidden_size)),
                  "o": ParamSpec((self.hidden_size, self.num_heads * self.value_dim))}
         if self.has_bias:
-            specs["qkv_bias"] = ParamSpec((self.q_size + self.k_size + self.v_size,), "float32", init=(0.0, 0.1))
+            specs["qkv_bias"] = ParamSpec((self.q_size + self.k_size + self.v_size,), "float32", init=(0.0, 0.02))
         if self.projection_norm_eps is not None:
             specs["q_norm"] = ParamSpec((self.q_size,), "float32", init=(1.0, 0.1))
             specs["k_norm"] = ParamSpec((self.k_size,), "float32", init=(1.0, 0.1))

@@ -58,9 +58,9 @@ class GatedDelta(Mixer):
         return StateSpec((self.sizes.matrix + self.sizes.kept,), torch.float32)
 
     def widest_activation(self) -> int:
-        # (a long portion's chunks of 64 tokens each keep four 64 x 64 tiles a head, and keys and values once more)
+        # (a long portion's chunks of 64 tokens each keep four 64 x 64 tiles a head, keys three times and values once more)
         z = self.sizes
-        return max(self.projected + 7, z.row, z.heads * (4 * hip.SSD_CHUNK + z.vp) + z.groups * z.np)
+        return max(self.projected + 7, z.row, z.heads * (4 * hip.SSD_CHUNK + z.vp) + 3 * z.groups * z.np)
 
     def keep_streaming_copies(self) -> int:
         self.proj_packed, self.o_packed = streaming_copy(self.proj), streaming_copy(self.o)
