@@ -1237,18 +1237,18 @@ def kufolorn_design(shape: str, layers: int | None):
                                          sh["intermediate_size"], sh["vocab_size"])
     # a delta rule of heads of 128, the values together twice as wide as the model and two heads to a key; beside attention of
     # the shape's heads over every position before, retention of heads of 128 as wide as the model; 16 experts of a quarter of
-    # the dense width and two identity experts in three groups of which two are kept, of which a token uses 4
-    dd, taps, experts, identity, groups, keep, top, eff = 128, 4, 16, 2, 3, 2, 4, inter // 4
+    # the dense width and four identity experts in five groups of which three are kept, of which a token uses 4
+    dd, taps, experts, identity, groups, keep, top, eff = 128, 4, 16, 4, 5, 3, 4, inter // 4
     dg, rh = hidden // dd, hidden // dd
     dh = 2 * dg
     decay = tuple(1.0 - 2.0 ** (-5.0 - 6.0 * i / max(1, rh - 1)) for i in range(rh))
     delta = KufolornDelta(heads=dh, kv_heads=dg, dim=dd, vdim=dd, conv=taps)
-    left = KufolornAttention(heads=nh, kv_heads=nkv, dim=hd, vdim=hd, scale=hd ** -0.5, rot=KufolornRotation(hd, 250000.0, 4.0))
+    left = KufolornAttention(heads=nh, kv_heads=nkv, dim=hd, vdim=hd, scale=hd ** -0.5, rot=KufolornRotation(hd, 500000.0, 2.0))
     right = KufolornRetention(heads=rh, dim=dd, vdim=dd, decay=decay, rot=KufolornRotation(dd, 10000.0))
-    par = KufolornParallel(left, right, left_scale=0.8, right_scale=0.9)
+    par = KufolornParallel(left, right, left_scale=0.7, right_scale=1.1)
     moe = KufolornExperts(experts=experts, identity=identity, top=top, ff=eff, limit=7.0, groups=groups, keep=keep)
     cycle = (("delta", delta, KufolornDense(inter)), ("parallel", par, moe)) * 2
-    kuf = KufolornConfig(vocab=vocab, width=hidden, norm_eps=1e-6, logit_softcap=30.0, layers=tuple(KufolornLayer(*cycle[i % 4]) for i in range(layers)))
+    kuf = KufolornConfig(vocab=vocab, width=hidden, norm_eps=1e-6, logit_softcap=20.0, layers=tuple(KufolornLayer(*cycle[i % 4]) for i in range(layers)))
     return kuf, dict(layers=layers, delta_heads=dh, delta_groups=dg, delta_dim=dd, conv_taps=taps, retention_heads=rh, retention_dim=dd, experts=experts,
                      identity=identity, groups=groups, keep=keep, top=top, eff=eff)
 
@@ -1335,7 +1335,7 @@ def kufolorn(args) -> int:
             x32, a32, w32 = torch.randn(T, hidden, device="cuda"), torch.randn(T, hidden, device="cuda"), torch.ones(hidden, device="cuda")
             entry("stream sum and norm", kufolorn=(timed(lambda: hip.stream_post_norm(x32, a32, w32, None, 1e-6, None, 0.0, bf)), T * hidden * (3 * 4 + 2)),
                   tegolix=(timed(lambda: hip.stream_post_norm(x32, a32, w32, w32, 1e-6, w32, 1e-6, bf)), T * hidden * (3 * 4 + 2)))
-            entry("two sides' sum", kufolorn=(timed(lambda: hip.scaled_sum(x32, 0.8, a32, 0.9)), T * hidden * 12))
+            entry("two sides' sum", kufolorn=(timed(lambda: hip.scaled_sum(x32, 0.7, a32, 1.1)), T * hidden * 12))
             # the unit of the dense feed-forward, the router, the logits' cap
             sums = torch.randn(T, 2 * inter, device="cuda")
             entry("gated unit", kufolorn=(timed(lambda: hip.capped_glu(sums, 0.0, 1.0, 0.0, bf, activation="gelu_tanh")), T * inter * 10),

@@ -258,7 +258,7 @@ def kufolorn_configs():
         L("delta", Dl(heads=3, kv_heads=1, dim=37, vdim=13, conv=6), D(52)),
         L("parallel", r_par, E(experts=5, identity=1, top=2, ff=17, limit=1.0, groups=2, keep=1))))
     # a width that the weight-streaming kernels take, heads of matrix-core sizes, experts in tiles of several rows
-    s_par = Par(A(heads=8, kv_heads=2, dim=64, vdim=64, scale=0.125, rot=Rot(64, 250000.0, 2.0)),
+    s_par = Par(A(heads=8, kv_heads=2, dim=64, vdim=64, scale=0.125, rot=Rot(64, 80000.0, 2.0)),
                 R(heads=4, dim=64, vdim=128, decay=(0.96, 0.99, 0.998, 0.9995), rot=Rot(64, 10000.0)), left_scale=0.9, right_scale=0.6)
     S = KufolornConfig(vocab=300, width=512, norm_eps=1e-6, logit_softcap=4.0, layers=(
         L("parallel", s_par, D(640)), L("delta", Dl(heads=8, kv_heads=4, dim=64, vdim=128, conv=4), E(experts=8, identity=2, top=4, ff=128, limit=1.2, groups=5, keep=3)),

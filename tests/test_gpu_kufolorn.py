@@ -193,7 +193,7 @@ def sink_case(dtype, H, G, D, V, page, length, queries, stand_out, portion_from,
 
 @pytest.mark.parametrize("form", sorted(FORMS))
 @pytest.mark.parametrize("dtype", DTYPES)
-@pytest.mark.parametrize("sizes", [(2, 2, 16, 16), (4, 2, 32, 48), (8, 2, 64, 64), (3, 1, 20, 12), (8, 4, 48, 48), (4, 1, 96, 96), (8, 4, 128, 128),
+@pytest.mark.parametrize("sizes", [(2, 2, 16, 16), (4, 2, 32, 48), (8, 2, 64, 64), (3, 1, 20, 12), (10, 5, 48, 48), (4, 1, 96, 96), (8, 4, 128, 128),
                                    (16, 2, 32, 32), (4, 4, 64, 1)])
 def test_sinks_and_gates_with_far_keys(dtype, sizes, form):
     """Far keys and keys at page borders stand out for their queries and decide their rows, beside a sink per head that
